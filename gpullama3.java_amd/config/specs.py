@@ -93,6 +93,21 @@ class DistanceBias:
 
 
 @dataclass(frozen=True)
+class QueryTemperature:
+    """The query at position p is multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)``."""
+    coef: float = 0.0
+    every: int = 1
+
+
+@dataclass(frozen=True)
+class ValueMix:
+    """Values blended across layers: of the layers that carry a ``ValueMix``, the one with ``first`` hands out its
+    values as projected, and every later one caches ``(1 - lambda) v + lambda v_first`` of the same token, ``lambda`` the
+    stored number ``v_mix`` among the attention's names. All of them have the same value heads and sizes."""
+    first: bool = False
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
     """Causal grouped-query attention over a cache of keys and values. Names ``q_bias``, ``k_bias``,
     ``v_bias`` (together) and ``o_bias`` among ``names`` add biases to the projections."""
@@ -121,6 +136,11 @@ class AttentionSpec:
     differential: Optional[Differential] = None
     values_are_keys: bool = False     # no value projection: a position's values are its keys as projected (before the
                                       # norm on keys and the rotation); ``names`` then has no ``v``
+    score_softcap: Optional[float] = None     # the scaled score becomes cap * tanh(score / cap), before any distance bias is taken off
+    query_temperature: Optional[QueryTemperature] = None
+    value_mix: Optional[ValueMix] = None
+    # (a name ``gate`` among ``names``: a stored [n_heads * v_head_dim, hidden] matrix; the heads' outputs together are
+    # multiplied element by element with sigmoid of its product with the mixer's input, before the output projection)
     # (a name ``sink`` among ``names``: a stored [n_heads] vector, a learned sink per query head in place of ``sink``)
     # (no ``k`` among ``names``: the mixer has no keys and values of its own and only ever reads another entry's)
     # (a name ``head_gate`` among ``names``: a stored [n_heads, hidden] matrix; head h's output is multiplied by
@@ -304,6 +324,11 @@ class RoutedFeedForwardSpec:
     sum_eps: float = 0.0
     n_identity: int = 0               # the router's last outputs stand for experts whose output is their input (no tensors);
                                       # the router has n_experts + n_identity rows
+    # A third rule (``weights = "sigmoid"``): the ``top`` largest router outputs are chosen, each weighted with its own
+    # sigmoid, not divided by anything. ``weight_on``: what the weight multiplies, the expert's "output" or its "input".
+    weight_on: str = "output"
+    # (a name ``shared_weight``: a stored [1, hidden] row; the shared expert's output is multiplied by sigmoid of its
+    # product with the token's input)
     # (names: ``expert_gate`` beside ``expert_up`` / ``expert_down`` for gated experts, ``shared_gate``; ``correction``)
 
 

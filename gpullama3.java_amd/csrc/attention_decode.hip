@@ -56,15 +56,15 @@ extern "C" int gl3_ad_stamps(long long* out) {
 // BIAS: a bias on the scores that grows with the distance, score - slopes[head] * (p - key), and a sink (a key
 // without a value that every query sees with the score `sink`; it joins the row sums where they are completed: here
 // with one split, in the merge kernel with several). A template parameter: the kernels without them are compiled
-// as they were.
-template <int HS, int NW, int CB, bool P2, bool BIAS = false>
+// as they were. RULE (with BIAS): the kernel also applies a Gl3ScoreRule (common.h).
+template <int HS, int NW, int CB, bool P2, bool BIAS = false, bool RULE = false>
 __global__ __launch_bounds__(NW * 64) void attention_decode_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ positions, const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
     int table_stride, float* __restrict__ part_o, float* __restrict__ part_ml, bf16_t* __restrict__ out,
     long out_stride, int n_heads, int n_kv, int g, int page_size, int page_shift, int window, float scale, int n_splits,
     const float* __restrict__ slopes, int has_sink, float sink, int keep_first, int mask_chunk, int maps,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, Gl3ScoreRule rule) {
   constexpr int KK = HS / 32;   // k-steps of the first product
   constexpr int DT = HS / 16;   // row tiles of the second product
   constexpr int NS = (HS > 64 && NW > 4) ? NW / 2 : NW;   // partial results that shared memory holds at a time
@@ -120,6 +120,25 @@ __global__ __launch_bounds__(NW * 64) void attention_decode_kernel(
     qt[kk] = j < heads_here ? *(const bf16x8*)(q + (long)t * q_stride + (long)(h0 + j * hstep) * HS + kk * 32 + 8 * qd) : zero8;
 
   const float slope = (BIAS && slopes && j < heads_here) ? slopes[h0 + j * hstep] : 0.f;
+  // (the gate's elements that this lane will need at the end are asked for here)
+  constexpr int GT = RULE ? (DT + NW - 1) / NW : 1;
+  bf16x4 gate_z[GT];
+  if (RULE && rule.gate && n_splits == 1) {
+#pragma unroll
+    for (int i = 0; i < GT; ++i) {
+      const int dt = min(wave + i * NW, DT - 1);
+      gate_z[i] = *(const bf16x4*)((const bf16_t*)rule.gate + (long)t * rule.gate_ld +
+                                   (long)(h0 + min(j, heads_here - 1) * hstep) * HS + dt * 16 + 4 * qd);
+    }
+  }
+  // a score is sum * scale, or with a rule sum * q_scale, or with a cap cap * tanh(sum * q_scale / cap)
+  const float q_scale = RULE ? scale * gl3_query_temperature(kv_len - 1, rule) : scale;
+  const float cap = RULE ? rule.softcap : 0.f;
+  const float cap_in = (RULE && cap > 0.f) ? 2.8853900817779268f * q_scale / cap : 0.f;
+  auto scored = [&](float sum) {
+    if (RULE && cap > 0.f) return cap * gl3_tanh_of_exponent(sum * cap_in);
+    return sum * q_scale;
+  };
   float m_run = -INFINITY, l_run = 0.f;   // l_run: this lane's share of the row sum
   f32x4 o[DT];
 #pragma unroll
@@ -171,8 +190,8 @@ __global__ __launch_bounds__(NW * 64) void attention_decode_kernel(
       for (int v = 0; v < 4; ++v) {
         const int ka_i = key0 + 8 * qd + v, kb_i = ka_i + 4;
         const float da = BIAS ? slope * (float)(kv_len - 1 - ka_i) : 0.f;     // (the bias: slope * distance; 4 keys on: 4 slopes less)
-        s[v] = ((ka_i >= lo || (BIAS && ka_i < keep_first)) && ka_i < kv_len) ? sa[v] * scale - da : -INFINITY;
-        s[4 + v] = ((kb_i >= lo || (BIAS && kb_i < keep_first)) && kb_i < kv_len) ? sb[v] * scale - (BIAS ? da - 4.f * slope : 0.f) : -INFINITY;
+        s[v] = ((ka_i >= lo || (BIAS && ka_i < keep_first)) && ka_i < kv_len) ? scored(sa[v]) - da : -INFINITY;
+        s[4 + v] = ((kb_i >= lo || (BIAS && kb_i < keep_first)) && kb_i < kv_len) ? scored(sb[v]) - (BIAS ? da - 4.f * slope : 0.f) : -INFINITY;
         mx = fmaxf(mx, fmaxf(s[v], s[4 + v]));
       }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -257,6 +276,14 @@ __global__ __launch_bounds__(NW * 64) void attention_decode_kernel(
     if (n_splits == 1) {
       bf16_t* op = out + (long)t * out_stride + (long)h * HS + dim;
       const float inv = 1.0f / L;
+      if (RULE && rule.gate) {
+        bf16x4 z = gate_z[0];
+#pragma unroll
+        for (int i = 1; i < GT; ++i)
+          if (dt >= i * NW) z = gate_z[i];
+#pragma unroll
+        for (int v = 0; v < 4; ++v) acc[v] *= gl3_sigmoid_fast((float)z[v]);
+      }
 #pragma unroll
       for (int v = 0; v < 4; ++v) op[v] = static_cast<bf16_t>(acc[v] * inv);
     } else {
@@ -278,7 +305,8 @@ __global__ __launch_bounds__(64) void attention_decode_merge_kernel(const float*
                                                                     const float* __restrict__ part_ml,
                                                                     bf16_t* __restrict__ out, long out_stride, int n_heads,
                                                                     int head_dim, int n_splits, int has_sink, float sink,
-                                                                    const float* __restrict__ sinks) {
+                                                                    const float* __restrict__ sinks,
+                                                                    const bf16_t* __restrict__ gate, long gate_ld) {
   const long th = blockIdx.x;   // token * n_heads + head
   const long t = th / n_heads, h = th % n_heads;
   if (sinks) {
@@ -322,6 +350,7 @@ __global__ __launch_bounds__(64) void attention_decode_merge_kernel(const float*
         acc += fs * v[e];
       }
     }
+    if (mine && gate) acc *= gl3_sigmoid_fast((float)gate[t * gate_ld + h * head_dim + d]);
     if (mine) out[t * out_stride + h * head_dim + d] = static_cast<bf16_t>(acc / L);
   }
 }
@@ -337,7 +366,8 @@ extern "C" int gl3_attention_decode(const void* q, long q_stride, const void* k_
                                     int table_stride, float* part_o, float* part_ml, long part_floats, void* out,
                                     long out_stride, int n_tokens, int n_heads, int n_kv, int head_dim, int page_size,
                                     int window, float scale, int n_splits, const float* slopes, int has_sink, float sink,
-                                    int keep_first, int mask_chunk, int maps, const float* sinks, hipStream_t stream) {
+                                    int keep_first, int mask_chunk, int maps, const float* sinks, float softcap,
+                                    float temp_coef, int temp_every, const void* gate, long gate_ld, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(q && k_cache && v_cache && positions && block_table && out && table_stride > 0,
               "gl3_attention_decode: null argument");
@@ -366,15 +396,25 @@ extern "C" int gl3_attention_decode(const void* q, long q_stride, const void* k_
   // first to end (what a block does before its keys arrive is a chain of trips to memory, paid once per round).
   const bool small = blocks * n_splits > 256;
   GL3_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "gl3_attention_decode: %d kept first keys without a window", keep_first);
+  const Gl3ScoreRule rule{softcap, temp_coef, temp_every, gate, gate_ld};
+  GL3_CHECK_RULE(rule, "gl3_attention_decode");
+  GL3_REQUIRE(!gate || (gate_ld % 4 == 0 && (uintptr_t)gate % 8 == 0), "gl3_attention_decode: gate rows must be 8-byte aligned");
+  const bool ruled = rule.any();
   const bool biased = slopes != nullptr || has_sink || sinks != nullptr || keep_first > 0;    // (the kernels that know of kept first keys)
 #define AD_ARGS                                                                                                       \
   (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, positions, seq_of_token, block_table,    \
       table_stride, part_o, part_ml, (bf16_t*)out, out_stride, n_heads, n_kv, n_heads / n_kv, page_size, page_shift, window,  \
-      scale, n_splits, slopes, has_sink, sink, keep_first, mask_chunk, maps, sinks
+      scale, n_splits, slopes, has_sink, sink, keep_first, mask_chunk, maps, sinks, rule
 #define GO(HS)                                                                                                        \
   do {                                                                                                                \
     constexpr int CB = HS <= 64 ? 4 : HS <= 96 ? 3 : 2;                                                               \
-    if (biased) {                                                                                                     \
+    if (ruled) {                                                                                                      \
+      if (small && p2) attention_decode_kernel<HS, 4, CB, true, true, true><<<grid, dim3(256), 0, stream>>>(AD_ARGS);  \
+      else if (small) attention_decode_kernel<HS, 4, CB, false, true, true><<<grid, dim3(256), 0, stream>>>(AD_ARGS);  \
+      else if (p2) attention_decode_kernel<HS, 8, CB, true, true, true><<<grid, dim3(512), 0, stream>>>(AD_ARGS);      \
+      else attention_decode_kernel<HS, 8, CB, false, true, true><<<grid, dim3(512), 0, stream>>>(AD_ARGS);             \
+    }                                                                                                                 \
+    else if (biased) {                                                                                                \
       if (small && p2) attention_decode_kernel<HS, 4, CB, true, true><<<grid, dim3(256), 0, stream>>>(AD_ARGS);        \
       else if (small) attention_decode_kernel<HS, 4, CB, false, true><<<grid, dim3(256), 0, stream>>>(AD_ARGS);        \
       else if (p2) attention_decode_kernel<HS, 8, CB, true, true><<<grid, dim3(512), 0, stream>>>(AD_ARGS);            \
@@ -396,7 +436,8 @@ extern "C" int gl3_attention_decode(const void* q, long q_stride, const void* k_
   GL3_LAUNCH_CHECK();
   if (n_splits > 1) {
     attention_decode_merge_kernel<<<dim3((unsigned)((long)n_tokens * n_heads)), dim3(64), 0, stream>>>(
-        part_o, part_ml, (bf16_t*)out, out_stride, n_heads, head_dim, n_splits, has_sink, sink, sinks);
+        part_o, part_ml, (bf16_t*)out, out_stride, n_heads, head_dim, n_splits, has_sink, sink, sinks,
+        (const bf16_t*)gate, gate_ld);
     GL3_LAUNCH_CHECK();
   }
   return 0;

@@ -22,7 +22,9 @@
 // ...]: query head h is map h % maps of head h / maps, which reads key head g * maps + h % maps and value head g, g the
 // head's group. The sink may be a number per query head (sinks). And values that are a part of the keys (v_in_k >= 0): a
 // cache with one array per position, whose elements v_in_k .. v_in_k + v_head_dim are the values (an attention over
-// cached latents); heads of up to 1024 elements then (MAXHS 1024: more registers, so a kernel of its own).
+// cached latents); heads of up to 1024 elements then (MAXHS 1024: more registers, so a kernel of its own). And what
+// Gl3ScoreRule (common.h) holds: a factor on the query that grows with its position, a soft cap on the scores in front
+// of the bias, a gate per element of the output.
 #include "common.h"
 
 #define ATT_MAX_HS 256
@@ -33,7 +35,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
     const int* __restrict__ positions, const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
     int table_stride, TO* __restrict__ out, long out_stride, int n_heads, int n_kv, int head_dim, int v_head_dim,
     int page_size, int window, float scale, const float* __restrict__ slopes, int has_sink, float sink, int keep_first,
-    int chunk, int n_v, const float* __restrict__ sinks, int v_in_k) {
+    int chunk, int n_v, const float* __restrict__ sinks, int v_in_k, Gl3ScoreRule rule) {
   __shared__ float qs[MAXHS];
   __shared__ float ps[64];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -47,6 +49,7 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
   for (int i = lane; i < head_dim; i += 64) qs[i] = to_f32<T>(qp[i]);
   __syncthreads();
   const float slope = slopes ? slopes[h] : 0.f;
+  const float q_scale = scale * gl3_query_temperature(p, rule);
   if (sinks) {
     has_sink = 1;
     sink = sinks[h];
@@ -67,7 +70,9 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
       const int in_page = key % page_size;
       float dot = 0.f;
       for (int i = 0; i < head_dim; ++i) dot = fmaf(qs[i], to_f32<T>(kp[gl3_k_offset(in_page, i, head_dim)]), dot);
-      s = dot * scale - slope * (float)(p - key);
+      s = dot * q_scale;
+      if (rule.softcap > 0.f) s = rule.softcap * tanhf(s / rule.softcap);
+      s = s - slope * (float)(p - key);
     }
     const float m_new = fmaxf(m, wave_max(s));
     const float pe = valid ? expf(s - m_new) : 0.f;
@@ -108,7 +113,14 @@ __global__ __launch_bounds__(64) void attention_generic_kernel(
 #pragma unroll
   for (int r = 0; r < MAXHS / 64; ++r) {
     const int i = lane + 64 * r;
-    if (i < v_head_dim) op[i] = from_f32<TO>(acc[r] / l);
+    if (i < v_head_dim) {
+      float v = acc[r] / l;
+      if (rule.gate) {
+        const float z = to_f32<T>(((const T*)rule.gate)[(long)t * rule.gate_ld + (long)h * v_head_dim + i]);
+        v *= 1.0f / (1.0f + expf(-z));
+      }
+      op[i] = from_f32<TO>(v);
+    }
   }
 }
 
@@ -117,7 +129,8 @@ extern "C" int gl3_attention_generic(const void* q, long q_stride, const void* k
                                      int table_stride, void* out, long out_stride, int n_tokens, int n_heads, int n_kv,
                                      int head_dim, int page_size, int window, float scale, int v_head_dim,
                                      const float* slopes, int has_sink, float sink, int keep_first, int chunk, int n_v,
-                                     int out_dtype, const float* sinks, int v_in_k, hipStream_t stream) {
+                                     int out_dtype, const float* sinks, int v_in_k, float softcap, float temp_coef,
+                                     int temp_every, const void* gate, long gate_ld, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(q && k_cache && (v_cache || v_in_k >= 0) && positions && seq_of_token && block_table && out,
               "gl3_attention_generic: null argument");
@@ -138,12 +151,14 @@ extern "C" int gl3_attention_generic(const void* q, long q_stride, const void* k
   GL3_REQUIRE(page_size % 32 == 0 && head_dim % 16 == 0,
               "gl3_attention_generic: the cache lies in tiles: page_size %d must be a multiple of 32, head_dim %d of 16", page_size,
               head_dim);
+  const Gl3ScoreRule rule{softcap, temp_coef, temp_every, gate, gate_ld};
+  GL3_CHECK_RULE(rule, "gl3_attention_generic");
   dim3 grid(n_tokens, n_heads), block(64);
 #define ATT_GENERIC_OF(T, TO, MAXHS)                                                                                   \
   attention_generic_kernel<T, TO, MAXHS><<<grid, block, 0, stream>>>(                                                  \
       (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, positions, seq_of_token, block_table, table_stride, \
       (TO*)out, out_stride, n_heads, n_kv, head_dim, v_head_dim, page_size, window, scale, slopes, has_sink, sink,     \
-      keep_first, chunk, n_v, sinks, v_in_k)
+      keep_first, chunk, n_v, sinks, v_in_k, rule)
 #define ATT_GENERIC(T, TO)                                                       \
   do {                                                                           \
     if (head_dim <= ATT_MAX_HS && v_head_dim <= ATT_MAX_HS) ATT_GENERIC_OF(T, TO, ATT_MAX_HS); \

@@ -40,14 +40,16 @@ __device__ __forceinline__ float max_over_quarters(float x) {
 
 // BIAS (both kernels): a bias on the scores that grows with the distance, score - slopes[head] * (p - key), and a
 // sink (a key without a value that every query sees with the score `sink`: the running softmax starts from it
-// instead of from nothing). A template parameter: the kernels without them are compiled as they were.
-template <int HS, int GH, bool BIAS = false>
+// instead of from nothing). A template parameter: the kernels without them are compiled as they were. RULE (with BIAS):
+// a Gl3ScoreRule (common.h); each score is then brought into units of log2 by itself, bias and all, where without
+// a rule the scale rides in the exponential.
+template <int HS, int GH, bool BIAS = false, bool RULE = false>
 __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ cu_seqlens, const int* __restrict__ kv_before, const int* __restrict__ block_table,
     const int* __restrict__ seq_rows, int table_stride, bf16_t* __restrict__ out, long out_stride, int n_heads, int n_kv, int page_size, int window,
     float scale, int q_blocks, const float* __restrict__ slopes, int has_sink, float sink, int keep_first, int mask_chunk, int maps,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, Gl3ScoreRule rule) {
   constexpr int KK = HS / 32;
   constexpr int DT = HS / 16;
   constexpr int KROW = HS + 8;            // a key row in shared memory, in elements
@@ -125,7 +127,8 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
   }
   float sl[GH];                                 // the heads' slopes over the scale: the scores are scaled afterwards
 #pragma unroll
-  for (int hh = 0; hh < GH; ++hh) sl[hh] = (BIAS && slopes && hh < heads_here) ? slopes[head_at(hh)] / scale : 0.f;
+  for (int hh = 0; hh < GH; ++hh)
+    sl[hh] = (BIAS && slopes && hh < heads_here) ? slopes[head_at(hh)] * (RULE ? 1.4426950408889634f : 1.0f / scale) : 0.f;
 
   // cache -> registers -> shared memory, 16 bytes a unit: a chunk's keys are 32 consecutive rows
   // of a page, its values 32 consecutive positions of each of the HS rows of the transposed page.
@@ -164,7 +167,10 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
     }
   };
 
-  const float c2 = scale * 1.4426950408889634f;   // scores in units of log2
+  const float c2 = RULE ? 1.0f : scale * 1.4426950408889634f;   // scores in units of log2
+  const float q_scale = RULE ? scale * gl3_query_temperature(p_mine, rule) : 0.f;
+  const float cap2 = RULE ? rule.softcap * 1.4426950408889634f : 0.f;      // the cap in units of log2
+  const float rule_in = !RULE ? 0.f : cap2 > 0.f ? 2.8853900817779268f * q_scale / rule.softcap : q_scale * 1.4426950408889634f;
   const int krow = 8 * (j >> 2) + (j & 3);   // which key of a chunk is row j of the first score tile
 
   // one chunk of one head: scores, running softmax, weighted values. MASKED: some query of the
@@ -182,6 +188,10 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
     for (int v = 0; v < 4; ++v) {
       s[v] = sa[v];
       s[4 + v] = sb[v];
+    }
+    if (RULE) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s[e] = cap2 > 0.f ? cap2 * gl3_tanh_of_exponent(s[e] * rule_in) : s[e] * rule_in;
     }
     if (BIAS) {
 #pragma unroll
@@ -270,6 +280,12 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       bf16x4 r;
+      if (RULE && rule.gate) {
+        const bf16x4 z = *(const bf16x4*)((const bf16_t*)rule.gate + (long)(tok0 + qi0 + j) * rule.gate_ld +
+                                          (long)head_at(hh) * HS + 4 * qd + dt * 16);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) o[hh][dt][v] *= gl3_sigmoid_fast((float)z[v]);
+      }
 #pragma unroll
       for (int v = 0; v < 4; ++v) r[v] = static_cast<bf16_t>(o[hh][dt][v] * inv);
       *(bf16x4*)(op + dt * 16) = r;
@@ -290,13 +306,13 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
 // its 16 keys a step.
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
-template <int HS, int CK, int AHEAD, int OCC, bool BIAS = false>
+template <int HS, int CK, int AHEAD, int OCC, bool BIAS = false, bool RULE = false>
 __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ cu_seqlens, const int* __restrict__ kv_before, const int* __restrict__ block_table,
     const int* __restrict__ seq_rows, int table_stride, bf16_t* __restrict__ out, long out_stride, int n_heads, int n_kv, int page_size, int window,
     float scale, int q_blocks, const float* __restrict__ slopes, int has_sink, float sink, int keep_first, int mask_chunk, int maps,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, Gl3ScoreRule rule) {
   constexpr int KS = HS / 16;             // steps of the score product
   constexpr int DT = HS / 32;             // tiles of 32 dims of the output
   constexpr int NT = CK / 32;             // score tiles of a chunk of CK keys
@@ -353,7 +369,7 @@ __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
     m_run = (sinks ? sinks[head] : sink) * 1.4426950408889634f;
     l_run = h == 0 ? 1.f : 0.f;
   }
-  const float sl = (BIAS && slopes) ? slopes[head] / scale : 0.f;
+  const float sl = (BIAS && slopes) ? slopes[head] * (RULE ? 1.4426950408889634f : 1.0f / scale) : 0.f;
   f32x16 o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
@@ -393,7 +409,10 @@ __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
     }
   };
 
-  const float c2 = scale * 1.4426950408889634f;   // scores in units of log2
+  const float c2 = RULE ? 1.0f : scale * 1.4426950408889634f;   // scores in units of log2
+  const float q_scale = RULE ? scale * gl3_query_temperature(p_mine, rule) : 0.f;
+  const float cap2 = RULE ? rule.softcap * 1.4426950408889634f : 0.f;      // the cap in units of log2
+  const float rule_in = !RULE ? 0.f : cap2 > 0.f ? 2.8853900817779268f * q_scale / rule.softcap : q_scale * 1.4426950408889634f;
   // which key of a chunk is row n of the score tile
   const int krow = 16 * (n >> 4) + 8 * ((n >> 2) & 1) + 4 * ((n >> 3) & 1) + (n & 3);
 
@@ -415,6 +434,13 @@ __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
         s[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, qt[kk], s[t], 0, 0, 0);
       }
       if (kk % 4 == 3) __builtin_amdgcn_sched_barrier(0);
+    }
+    if (RULE) {
+#pragma unroll
+      for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int v = 0; v < 16; ++v)
+          s[t][v] = cap2 > 0.f ? cap2 * gl3_tanh_of_exponent(s[t][v] * rule_in) : s[t][v] * rule_in;
     }
     if (BIAS) {
 #pragma unroll
@@ -511,6 +537,12 @@ __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
 #pragma unroll
     for (int a = 0; a < 4; ++a) {
       bf16x4 r;
+      if (RULE && rule.gate) {
+        const bf16x4 z = *(const bf16x4*)((const bf16_t*)rule.gate + (long)(tok0 + qi0 + n) * rule.gate_ld +
+                                          (long)head * HS + 4 * h + dt * 32 + 8 * a);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) o[dt][4 * a + v] *= gl3_sigmoid_fast((float)z[v]);
+      }
 #pragma unroll
       for (int v = 0; v < 4; ++v) r[v] = static_cast<bf16_t>(o[dt][4 * a + v] * inv);
       *(bf16x4*)(op + dt * 32 + 8 * a) = r;
@@ -540,7 +572,8 @@ extern "C" int gl3_attention_prefill(const void* q, long q_stride, const void* k
                                      const int* seq_rows, int table_stride, void* out, long out_stride, int n_seqs,
                                      int max_q_len, int n_heads, int n_kv, int head_dim, int page_size, int window,
                                      float scale, int wide_from, const float* slopes, int has_sink, float sink,
-                                     int keep_first, int mask_chunk, int maps, const float* sinks, hipStream_t stream) {
+                                     int keep_first, int mask_chunk, int maps, const float* sinks, float softcap,
+                                     float temp_coef, int temp_every, const void* gate, long gate_ld, hipStream_t stream) {
   if (n_seqs == 0 || max_q_len == 0) return 0;
   GL3_REQUIRE(q && k_cache && v_cache && cu_seqlens && kv_before && block_table && out,
               "gl3_attention_prefill: null argument");
@@ -566,14 +599,19 @@ extern "C" int gl3_attention_prefill(const void* q, long q_stride, const void* k
               n_seqs, q_blocks);
   dim3 grid((unsigned)z, n_seqs, q_blocks), block(256);
   GL3_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "gl3_attention_prefill: %d kept first keys without a window", keep_first);
+  const Gl3ScoreRule rule{softcap, temp_coef, temp_every, gate, gate_ld};
+  GL3_CHECK_RULE(rule, "gl3_attention_prefill");
+  GL3_REQUIRE(!gate || (gate_ld % 4 == 0 && (uintptr_t)gate % 8 == 0), "gl3_attention_prefill: gate rows must be 8-byte aligned");
+  const bool ruled = rule.any();
   const bool biased = slopes != nullptr || has_sink || sinks != nullptr || keep_first > 0;    // (the kernels that know of kept first keys)
   if (wide) {
 #define PF_ARGS                                                                                                     \
   (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, cu_seqlens, kv_before, block_table,     \
-      seq_rows, table_stride, (bf16_t*)out, out_stride, n_heads, n_kv, page_size, window, scale, q_blocks, slopes, has_sink, sink, keep_first, mask_chunk, maps, sinks
+      seq_rows, table_stride, (bf16_t*)out, out_stride, n_heads, n_kv, page_size, window, scale, q_blocks, slopes, has_sink, sink, keep_first, mask_chunk, maps, sinks, rule
 #define GOW(HS, CK, AH, OCC)                                                                                        \
   do {                                                                                                              \
-    if (biased) attention_prefill_wide_kernel<HS, CK, AH, OCC, true><<<grid, block, 0, stream>>>(PF_ARGS);          \
+    if (ruled) attention_prefill_wide_kernel<HS, CK, AH, OCC, true, true><<<grid, block, 0, stream>>>(PF_ARGS);     \
+    else if (biased) attention_prefill_wide_kernel<HS, CK, AH, OCC, true><<<grid, block, 0, stream>>>(PF_ARGS);     \
     else attention_prefill_wide_kernel<HS, CK, AH, OCC, false><<<grid, block, 0, stream>>>(PF_ARGS);                \
   } while (0)
     // chunks of 64 keys (one barrier for twice the work, two score tiles whose sums do not wait for
@@ -591,7 +629,8 @@ extern "C" int gl3_attention_prefill(const void* q, long q_stride, const void* k
   }
 #define GO(HS, GH)                                                                                                  \
   do {                                                                                                              \
-    if (biased) attention_prefill_kernel<HS, GH, true><<<grid, block, 0, stream>>>(PF_ARGS);                        \
+    if (ruled) attention_prefill_kernel<HS, GH, true, true><<<grid, block, 0, stream>>>(PF_ARGS);                   \
+    else if (biased) attention_prefill_kernel<HS, GH, true><<<grid, block, 0, stream>>>(PF_ARGS);                   \
     else attention_prefill_kernel<HS, GH, false><<<grid, block, 0, stream>>>(PF_ARGS);                              \
   } while (0)
   switch (head_dim) {

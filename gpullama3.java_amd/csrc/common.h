@@ -153,6 +153,34 @@ __device__ __forceinline__ float gl3_activation(float v, int act) {
   return v / (1.0f + (FAST ? __expf(-v) : expf(-v)));
 }
 
+// What a description may do to attention scores and outputs beyond the plain rule (``lib.ScoreRule``): the query at
+// position p counts `1 + temp_coef ln(floor((p + 1) / temp_every) + 1)` times (temp_every 0: once); a score is bounded
+// to `softcap * tanh(score / softcap)` (softcap 0: not) before any bias that grows with the distance is taken off; and
+// the heads' outputs are multiplied by sigmoid of the gate rows' elements (gate null: not), row t at gate + t gate_ld,
+// the elements in the order of the output's.
+struct Gl3ScoreRule {
+  float softcap;
+  float temp_coef;
+  int temp_every;
+  const void* gate;
+  long gate_ld;
+  bool any() const { return softcap != 0.f || temp_every != 0 || gate != nullptr; }
+};
+#define GL3_CHECK_RULE(r, who)                                                                                       \
+  GL3_REQUIRE((r).softcap >= 0.f && (r).temp_every >= 0, who ": a soft cap of %g, a temperature that steps every %d", \
+              (double)(r).softcap, (r).temp_every)
+__device__ __forceinline__ float gl3_query_temperature(int p, const Gl3ScoreRule& r) {
+  return r.temp_every > 0 ? 1.0f + r.temp_coef * logf((float)((p + 1) / r.temp_every + 1)) : 1.0f;
+}
+// tanh by one exponential and one reciprocal: 1 - 2 / (1 + e^(2y)), given y2 = 2 y log2(e); its error is one of
+// 32-bit rounding of numbers around one (not relative to a small tanh).
+__device__ __forceinline__ float gl3_tanh_of_exponent(float y2) {
+  return fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(y2)), 1.0f);
+}
+__device__ __forceinline__ float gl3_sigmoid_fast(float z) {
+  return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+
 // The gated epilogue's rule in full: act(gate) * (up + shift), where a positive `limit` first bounds the
 // gate from above (min(gate, limit)) and the up value on both sides (clamp(up, -limit, limit)). The
 // reference's feed-forward is limit = 0 (none), shift = 0.

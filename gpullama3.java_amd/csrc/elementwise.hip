@@ -573,11 +573,14 @@ extern "C" int gl3_decode_advance(int* token_ids, int* positions, int* kv_before
 // Rows of a projection [T][ld] whose columns k_off .. hold n_kv keys of head_dim and v_off .. n_kv values of
 // v_head_dim go to the token's place in its page, unrotated: what an attention without a rotation, or with values
 // of another size than its keys, writes. grid (T, 2 n_kv): key heads, then value heads.
+// With `first` (rows [T][first_ld], value heads of first_dim one after another from column 0) the values are blended with
+// another layer's values of the same token on their way: (1 - mix) v + mix first; elements beyond first_dim count as 0.
 template <typename T>
 __global__ void kv_write_kernel(const T* __restrict__ rows, long ld, int k_off, int v_off,
                                 const int* __restrict__ positions, const int* __restrict__ table_rows,
                                 const int* __restrict__ block_table, int table_stride, T* __restrict__ k_cache,
-                                T* __restrict__ v_cache, int n_kv, int head_dim, int v_head_dim, int page_size) {
+                                T* __restrict__ v_cache, int n_kv, int head_dim, int v_head_dim, int page_size,
+                                const T* __restrict__ first, long first_ld, int first_dim, float mix) {
   const int t = blockIdx.x, u = blockIdx.y;
   const int pos = positions[t];
   const long page = block_table[(long)table_rows[t] * table_stride + pos / page_size];
@@ -590,14 +593,87 @@ __global__ void kv_write_kernel(const T* __restrict__ rows, long ld, int k_off, 
     const int c = u - n_kv;
     const T* src = rows + (long)t * ld + v_off + (long)c * v_head_dim;
     T* vpage = v_cache + (page * n_kv + c) * page_size * v_head_dim;
-    for (int i = threadIdx.x; i < v_head_dim; i += blockDim.x) vpage[gl3_v_offset(i, in_page, page_size)] = src[i];
+    const T* other = first ? first + (long)t * first_ld + (long)c * first_dim : nullptr;
+    for (int i = threadIdx.x; i < v_head_dim; i += blockDim.x) {
+      T v = src[i];
+      if (other) v = from_f32<T>((1.0f - mix) * to_f32<T>(v) + mix * (i < first_dim ? to_f32<T>(other[i]) : 0.f));
+      vpage[gl3_v_offset(i, in_page, page_size)] = v;
+    }
+  }
+}
+
+// The same for bfloat16 rows in units of 8 elements (16 bytes), a block a token. The values of 8 consecutive positions
+// share 16 bytes of a transposed page: the first of the step's tokens in such a group of 8 positions writes the values
+// of all of them that the step brings (they follow it in the packed order), whole groups as 16 bytes a dim. Blocks are
+// numbered so that neighbouring tokens go to one XCD's second-level cache (as rope_cache_vec_kernel does both).
+__global__ __launch_bounds__(256) void kv_write_vec_kernel(const bf16_t* __restrict__ rows, long ld, int k_off, int v_off,
+                                                           const int* __restrict__ positions,
+                                                           const int* __restrict__ table_rows,
+                                                           const int* __restrict__ block_table, int table_stride,
+                                                           bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache, int n_kv,
+                                                           int head_dim, int v_head_dim, int page_size, int n_tokens,
+                                                           const bf16_t* __restrict__ first, long first_ld, int first_dim,
+                                                           float mix) {
+  const int per_xcd = (n_tokens + 7) / 8;
+  const int t = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
+  if (t >= n_tokens) return;
+  const int pos = positions[t], seq = table_rows[t];
+  const long page = block_table[(long)seq * table_stride + pos / page_size];
+  const int in_page = pos % page_size;
+  const int kd = head_dim / 8, vd = v_head_dim / 8;         // units a head
+  int run = 0;                                             // how many tokens' values this block writes
+  if ((pos & 7) == 0 || t == 0 || table_rows[t - 1] != seq || positions[t - 1] != pos - 1) {
+    run = 1;
+    while (run < 8 - (pos & 7) && t + run < n_tokens && table_rows[t + run] == seq && positions[t + run] == pos + run) ++run;
+  }
+  const int total = n_kv * kd + (run ? n_kv * vd : 0);
+  for (int w = threadIdx.x; w < total; w += blockDim.x) {
+    if (w < n_kv * kd) {                        // a unit of a key head
+      const int c = w / kd, e0 = (w % kd) * 8;
+      bf16_t* kpage = k_cache + (page * n_kv + c) * (long)page_size * head_dim;
+      *(rc_bf16x8*)(kpage + gl3_k_offset(in_page, e0, head_dim)) =
+          *(const rc_bf16x8*)(rows + (long)t * ld + k_off + (long)c * head_dim + e0);
+      continue;
+    }
+    const int u = w - n_kv * kd, c = u / vd, e0 = (u % vd) * 8;
+    bf16_t* vat = v_cache + (page * n_kv + c) * (long)page_size * v_head_dim + gl3_v_offset(e0, in_page, page_size);
+    const bf16_t* from = rows + (long)t * ld + v_off + (long)c * v_head_dim + e0;
+    const bf16_t* other = first && e0 < first_dim ? first + (long)t * first_ld + (long)c * first_dim + e0 : nullptr;
+    auto value = [&](int i) {                    // the 8 elements of the token i further
+      rc_bf16x8 v = *(const rc_bf16x8*)(from + (long)i * ld);
+      if (first) {
+        rc_bf16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
+        if (other) f = *(const rc_bf16x8*)(other + (long)i * first_ld);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = static_cast<bf16_t>((1.0f - mix) * (float)v[e] + mix * (float)f[e]);
+      }
+      return v;
+    };
+    if (run == 8) {                              // a whole group of 8 positions (pos % 8 == 0)
+      rc_bf16x8 v[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] = value(i);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        rc_bf16x8 o;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = v[i][e];
+        *(rc_bf16x8*)(vat + 8 * e) = o;
+      }
+    } else {
+      for (int i = 0; i < run; ++i) {
+        const rc_bf16x8 v = value(i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) vat[i + 8 * e] = v[e];
+      }
+    }
   }
 }
 
 extern "C" int gl3_kv_write(const void* rows, int dtype, long ld, int k_off, int v_off, const int* positions,
                             const int* table_rows, const int* block_table, int table_stride, void* k_cache,
                             void* v_cache, int n_tokens, int n_kv, int head_dim, int v_head_dim, int page_size,
-                            hipStream_t stream) {
+                            const void* first, long first_ld, int first_dim, float mix, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(rows && positions && table_rows && block_table && k_cache && v_cache && n_tokens > 0 && n_kv > 0 &&
                   table_stride > 0, "gl3_kv_write: bad arguments");
@@ -607,15 +683,29 @@ extern "C" int gl3_kv_write(const void* rows, int dtype, long ld, int k_off, int
               page_size, head_dim, v_head_dim);
   GL3_REQUIRE(k_off >= 0 && v_off >= 0 && k_off + (long)n_kv * head_dim <= ld && v_off + (long)n_kv * v_head_dim <= ld &&
                   2 * n_kv <= 65535, "gl3_kv_write: columns %d and %d of rows of %ld", k_off, v_off, ld);
+  GL3_REQUIRE(!first || (first_dim > 0 && (long)n_kv * first_dim <= first_ld),
+              "gl3_kv_write: %d other values of %d in rows of %ld", n_kv, first_dim, first_ld);
+  // bfloat16 rows whose places allow 16-byte units take the kernel of one block a token
+  if (dtype == GL3_BF16 && ld % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && (uintptr_t)rows % 16 == 0 &&
+      (uintptr_t)k_cache % 16 == 0 && (uintptr_t)v_cache % 16 == 0 &&
+      (!first || (first_ld % 8 == 0 && first_dim % 8 == 0 && (uintptr_t)first % 16 == 0))) {
+    kv_write_vec_kernel<<<dim3((n_tokens + 7) / 8 * 8), dim3(256), 0, stream>>>(
+        (const bf16_t*)rows, ld, k_off, v_off, positions, table_rows, block_table, table_stride, (bf16_t*)k_cache,
+        (bf16_t*)v_cache, n_kv, head_dim, v_head_dim, page_size, n_tokens, (const bf16_t*)first, first_ld, first_dim, mix);
+    GL3_LAUNCH_CHECK();
+    return 0;
+  }
   dim3 grid(n_tokens, 2 * n_kv), block(64);
   if (dtype == GL3_F32)
     kv_write_kernel<float><<<grid, block, 0, stream>>>((const float*)rows, ld, k_off, v_off, positions, table_rows,
                                                        block_table, table_stride, (float*)k_cache, (float*)v_cache, n_kv,
-                                                       head_dim, v_head_dim, page_size);
+                                                       head_dim, v_head_dim, page_size, (const float*)first, first_ld,
+                                                       first_dim, mix);
   else if (dtype == GL3_BF16)
     kv_write_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)rows, ld, k_off, v_off, positions, table_rows,
                                                         block_table, table_stride, (bf16_t*)k_cache, (bf16_t*)v_cache,
-                                                        n_kv, head_dim, v_head_dim, page_size);
+                                                        n_kv, head_dim, v_head_dim, page_size, (const bf16_t*)first,
+                                                        first_ld, first_dim, mix);
   else GL3_REQUIRE(false, "gl3_kv_write: unknown dtype %d", dtype);
   GL3_LAUNCH_CHECK();
   return 0;

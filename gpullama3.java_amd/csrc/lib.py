@@ -9,6 +9,7 @@ from __future__ import annotations
 
 import ctypes
 from ctypes import c_float, c_int, c_long, c_uint32, c_void_p
+from typing import NamedTuple, Optional
 
 import torch
 
@@ -57,7 +58,7 @@ def _declare(lib):
         "gl3_add_slices_rmsnorm": [P, P, P, I, L, L, P, I, P, I, I, I, F, P],
         "gl3_rope_cache_write": [P, I, P, P, P, I, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "gl3_gemm_generic": [P, I, P, I, P, I, I, I, I, L, L, L, I, P, I, I, P, F, F, P, P],
-        "gl3_attention_generic": [P, L, P, P, I, P, P, P, I, P, L, I, I, I, I, I, I, F, I, P, I, F, I, I, I, I, P, I, P],
+        "gl3_attention_generic": [P, L, P, P, I, P, P, P, I, P, L, I, I, I, I, I, I, F, I, P, I, F, I, I, I, I, P, I, F, F, I, P, L, P],
         "gl3_pair_rows": [P, P, P, P, P, P, L, L, L, L, P, I, P],
         "gl3_concat_rows": [P, P, P, I, I, I, P],
         "gl3_rotate_heads": [P, I, L, P, I, P, P, P, P, P, P, I, I, I, P, L, I, P, P, P, P, I, I, P, P, F, P],
@@ -68,9 +69,9 @@ def _declare(lib):
         "gl3_ssm_prep": [P, L, I, I, I, I, I, I, P, P, I, P, P, P, L, L, P, P, P, P, P, P],
         "gl3_decay_scan": [P, L, I, P, L, I, P, L, I, P, P, L, P, F, P, L, L, P, P, P, L, I, I, I, I, I, P, L, I, I, I, P],
         "gl3_group_norm_gate": [P, P, L, I, P, I, P, L, I, P, F, I, I, I, I, P, I, I, P],
-        "gl3_route": [P, I, I, I, P, P, P, P, I, I, P, F, P],
-        "gl3_expert_gemm": [P, I, L, I, P, I, I, I, I, P, P, I, P, I, L, I, I, I, F, F, P],
-        "gl3_route_combine": [P, P, I, I, I, P, I, P, I, P, I, P],
+        "gl3_route": [P, I, I, I, P, P, P, P, I, I, P, F, I, P, I, P, P, I, I, F, P, P],
+        "gl3_expert_gemm": [P, I, L, I, P, I, I, I, I, P, P, I, P, I, L, I, I, I, F, F, P, P, P],
+        "gl3_route_combine": [P, P, I, I, I, P, I, P, I, P, I, P, P, P, P],
         "gl3_streams_step": [P, I, I, I, P, P, P, P, P, F, P, I, P],
         "gl3_streams_fill": [P, P, I, I, I, P],
         "gl3_streams_sum": [P, P, I, I, I, P, P],
@@ -85,7 +86,7 @@ def _declare(lib):
         "gl3_shift_mix": [P, I, I, P, I, P, L, P, P, P, P, I, I, I, P],
         "gl3_timemix": [P, P, P, L, P, L, P, P, L, L, P, P, P, I, I, I, P, L, P, F, P, I, I, P],
         "gl3_head_norm_gate": [P, P, P, F, P, I, I, I, I, P],
-        "gl3_kv_write": [P, I, L, I, I, P, P, P, I, P, P, I, I, I, I, I, P],
+        "gl3_kv_write": [P, I, L, I, I, P, P, P, I, P, P, I, I, I, I, I, P, L, I, F, P],
         "gl3_residual_inject": [P, P, P, I, I, P],
         "gl3_delta_state_floats": [I, I, I, I, I],
         "gl3_delta_prep": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, I, L, F, F, I, P],
@@ -104,13 +105,13 @@ def _declare(lib):
         "gl3_gemm_mfma": [P, P, P, I, I, I, I, L, L, L, I, I, P, L, L, P, I, I, I, P, F, F, P, P],
         "gl3_attention_decode_supports": [I, I],
         "gl3_attention_prefill_supports": [I, I],
-        "gl3_attention_prefill": [P, L, P, P, P, P, P, P, I, P, L, I, I, I, I, I, I, I, F, I, P, I, F, I, I, I, P, P],
+        "gl3_attention_prefill": [P, L, P, P, P, P, P, P, I, P, L, I, I, I, I, I, I, I, F, I, P, I, F, I, I, I, P, F, F, I, P, L, P],
         "gl3_scatter_i32": [P, L, P, P, I, P],
         "gl3_upload": [P, P, L, P],
         "gl3_stage_decode": [P, I, I, P, P, P, I, P, P],
         "gl3_stage_step": [P, P, P, I, P, P, P, I, P, I, I, P],
         "gl3_graph_launch": [P, P],
-        "gl3_attention_decode": [P, L, P, P, P, P, P, I, P, P, L, P, L, I, I, I, I, I, I, F, I, P, I, F, I, I, I, P, P],
+        "gl3_attention_decode": [P, L, P, P, P, P, P, I, P, P, L, P, L, I, I, I, I, I, I, F, I, P, I, F, I, I, I, P, F, F, I, P, L, P],
     }
     for name, args in sigs.items():
         fn = getattr(lib, name, None)
@@ -254,6 +255,32 @@ def _sink(sink, n_heads, who):
             raise KernelError(f"{who}: {tuple(sink.shape)} sinks for {n_heads} heads")
         return 0, 0.0, _ptr(sink)
     return 1, float(sink), None
+
+
+class ScoreRule(NamedTuple):
+    """What a description may do to attention scores and outputs beyond the plain rule. ``temperature = (coef, every)``:
+    the query at position p counts ``1 + coef ln(floor((p + 1) / every) + 1)`` times; ``softcap``: a score becomes
+    ``softcap * tanh(score / softcap)`` in front of the distance bias and the mask; ``gate``: rows [T, n_heads * values' size]
+    of the queries' type (a view of wider rows), whose sigmoids multiply the heads' outputs element by element."""
+    softcap: Optional[float] = None
+    temperature: Optional[tuple] = None
+    gate: Optional[torch.Tensor] = None
+
+
+def _rule(rule, T, columns, dtype, who):
+    """A ``ScoreRule`` (or None) as the kernels take it."""
+    if rule is None:
+        return 0.0, 0.0, 0, None, 0
+    coef, every = rule.temperature if rule.temperature is not None else (0.0, 0)
+    if rule.softcap is not None and not rule.softcap > 0 or rule.temperature is not None and every < 1:
+        raise KernelError(f"{who}: a soft cap of {rule.softcap}, a temperature of {rule.temperature}")
+    gate, ld = rule.gate, 0
+    if gate is not None:
+        _dev(gate, "gate", dtype, contiguous=False)
+        if gate.shape != (T, columns) or gate.stride(1) != 1:
+            raise KernelError(f"{who}: gate rows {tuple(gate.shape)} for outputs [{T}, {columns}]")
+        ld = gate.stride(0)
+    return float(rule.softcap or 0.0), float(coef), int(every), _ptr(gate), ld
 
 
 def _act(act, who):
@@ -422,8 +449,8 @@ def gemm_generic(a, w, out, epilogue=EPI_STORE, bias=None, act="silu", act_limit
 
 def attention_generic(q, k_cache, v_cache, positions, seq_of_token, block_table, out, n_heads, n_kv, head_dim,
                       page_size, window, scale, v_head_dim=None, slopes=None, sink=None, keep_first=0, chunk=0, n_v_heads=None,
-                      values_in_keys=None):
-    """``sink`` may also be a float32 tensor [H]: a sink per query head. ``values_in_keys``: n: the cache has no value
+                      values_in_keys=None, rule=None):
+    """``rule``: a ``ScoreRule``. ``sink`` may also be a float32 tensor [H]: a sink per query head. ``values_in_keys``: n: the cache has no value
     array (``v_cache`` None); the values are elements n .. n + v_head_dim of the key rows (heads of up to 1024).
     q: a [T, >= H*hs] view whose first H*hs columns of each row are the queries. ``v_head_dim``: the values'
     size where it is not the keys'; ``slopes``: float32 [H], score - slopes[h] * distance; ``sink``: the score of a
@@ -467,14 +494,17 @@ def attention_generic(q, k_cache, v_cache, positions, seq_of_token, block_table,
         _ptr(block_table), block_table.shape[1], _ptr(out), out.stride(0), T, n_heads, n_kv, head_dim, page_size,
         int(window or 0), float(scale), vd, _ptr(slopes), has_sink, sink_value,
         int(keep_first or 0) if window else 0, int(chunk or 0), n_v, _code(out, "out"), sinks,
-        -1 if values_in_keys is None else int(values_in_keys), _stream()),
+        -1 if values_in_keys is None else int(values_in_keys),
+        *_rule(rule, T, n_heads * vd, q.dtype, "attention"), _stream()),
         "attention_generic")
 
 
 def kv_write(rows, k_off, v_off, positions, table_rows, block_table, k_cache, v_cache, n_kv, head_dim, v_head_dim,
-             page_size):
+             page_size, blend=None):
     """Keys (columns ``k_off`` .. of ``rows`` [T, ld]) and values (``v_off`` ..) of the step's tokens into one
-    layer's paged cache, unrotated; the values may have another size than the keys."""
+    layer's paged cache, unrotated; the values may have another size than the keys. ``blend = (other, dim, mix)``: the
+    values become ``(1 - mix) v + mix other`` on their way, ``other`` rows [T, n_kv * dim] of the same type (a view of
+    wider rows) with heads of ``dim`` elements, of which what lies beyond counts as zero."""
     _dev(rows, "rows", contiguous=False); _dev(positions, "positions", torch.int32)
     _dev(table_rows, "table_rows", torch.int32); _dev(block_table, "block_table", torch.int32)
     _dev(k_cache, "k_cache", rows.dtype); _dev(v_cache, "v_cache", rows.dtype)
@@ -484,9 +514,17 @@ def kv_write(rows, k_off, v_off, positions, table_rows, block_table, k_cache, v_
     _check_cache(k_cache, v_cache, n_kv, page_size, head_dim, "kv_write", v_head_dim)
     if k_off < 0 or v_off < 0 or k_off + n_kv * head_dim > rows.shape[1] or v_off + n_kv * v_head_dim > rows.shape[1]:
         raise KernelError(f"kv_write: columns {k_off} and {v_off} of rows of {rows.shape[1]}")
+    other, other_ld, other_dim, mix = None, 0, 0, 0.0
+    if blend is not None:
+        other, other_dim, mix = blend[0], int(blend[1]), float(blend[2])
+        _dev(other, "other values", rows.dtype, contiguous=False)
+        if other.shape != (T, n_kv * other_dim) or other.stride(1) != 1:
+            raise KernelError(f"kv_write: other values {tuple(other.shape)} for {n_kv} heads of {other_dim}")
+        other_ld = other.stride(0)
     _check(library().gl3_kv_write(_ptr(rows), _code(rows, "rows"), rows.stride(0), k_off, v_off, _ptr(positions),
                                   _ptr(table_rows), _ptr(block_table), block_table.shape[1], _ptr(k_cache), _ptr(v_cache),
-                                  T, n_kv, head_dim, v_head_dim, page_size, _stream()), "kv_write")
+                                  T, n_kv, head_dim, v_head_dim, page_size, _ptr(other), other_ld, other_dim, mix, _stream()),
+           "kv_write")
 
 
 def residual_inject(x, rows=None, vec=None):
@@ -777,18 +815,28 @@ EXPERT_ACTIVATIONS = {None: 0, "gelu": 1, "gelu_tanh": 2, "silu": 3}
 ROUTE_MAX_TOP, ROUTE_MAX_EXPERTS = 16, 1024      # as csrc/routed.hip has them
 
 
-def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, correction=None, sum_eps=0.0):
+def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, correction=None, sum_eps=0.0, n_experts=None,
+          in_wts=None, gate_col=None, gate_out=None, norm=None, norm_out=None):
     """Router logits [T, E] float32 -> the ``top`` largest per token (``idx`` [T, top] int32, the lower number wins a
     tie) with the softmax over them alone (``wts`` [T, top]); and the (token, choice) pairs ordered by expert:
     ``offsets`` [E + 1] int32, ``pairs`` [T top] int32 (pair t * top + j). ``always``: every token has one more pair
     behind its choices, with expert number E and weight 1 (``idx`` and ``wts`` [T, top + 1], ``offsets`` [E + 2],
     ``pairs`` [T (top + 1)]). ``scores``: the other rule: s = softmax over all E logits, the choice goes by
-    s + ``correction`` (float32 [E], optional), the weights are the chosen s divided by their sum plus ``sum_eps``."""
+    s + ``correction`` (float32 [E], optional), the weights are the chosen s divided by their sum plus ``sum_eps``.
+    ``scores = "sigmoid"``: the third rule: the largest logits are chosen, their weights are their sigmoids.
+    ``n_experts``: the logits' first columns are the experts' (None: all are). ``in_wts`` (like ``wts``): the weights belong
+    to the experts' inputs: they go here, and ``wts`` takes what the outputs count (1). ``gate_col``: the column of logits
+    whose sigmoid multiplies the output of the expert that every token passes: into ``wts`` where that expert has pairs
+    (``always``), and to ``gate_out`` [T] where given. ``norm = (ssq, n_partials, d, eps)`` (at most 64 tokens, with
+    ``in_wts``): the rows that the experts multiply lack their 1 / rms, which is made from the partial sums of squares,
+    rides in ``in_wts`` and goes to ``norm_out`` [T] where given."""
     _dev(logits, "logits", torch.float32)
-    T, E = logits.shape
+    T, ld = logits.shape
+    E = ld if n_experts is None else int(n_experts)
+    rule = 2 if scores == "sigmoid" else int(bool(scores))
     if correction is not None:
         _dev(correction, "correction", torch.float32)
-        if not scores or correction.shape != (E,):
+        if rule != 1 or correction.shape != (E,):
             raise KernelError(f"route: a correction {tuple(correction.shape)} for {E} scores")
     more = 1 if always else 0
     for t, name, shape, dt in ((idx, "idx", (T, top + more), torch.int32), (wts, "wts", (T, top + more), torch.float32),
@@ -797,17 +845,31 @@ def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, cor
         _dev(t, name, dt)
         if tuple(t.shape) != shape:
             raise KernelError(f"route: {name} {tuple(t.shape)}, expected {shape}")
+    for t, name, shape in ((in_wts, "in_wts", (T, top + more)), (gate_out, "gate_out", (T,)), (norm_out, "norm_out", (T,))):
+        if t is not None:
+            _dev(t, name, torch.float32)
+            if tuple(t.shape) != shape:
+                raise KernelError(f"route: {name} {tuple(t.shape)}, expected {shape}")
+    ssq, n_partials, d, eps = norm if norm is not None else (None, 0, 0, 0.0)
+    if ssq is not None:
+        _dev(ssq, "ssq", torch.float32)
+        if T > 64 or ssq.numel() < n_partials * 64:
+            raise KernelError(f"route: {n_partials} x 64 partial sums of squares for {T} tokens, {ssq.numel()} given")
     _check(library().gl3_route(_ptr(logits), T, E, int(top), _ptr(idx), _ptr(wts), _ptr(offsets), _ptr(pairs),
-                               E if always else -1, int(bool(scores)), _ptr(correction), float(sum_eps), _stream()), "route")
+                               E if always else -1, rule, _ptr(correction), float(sum_eps), ld, _ptr(in_wts),
+                               -1 if gate_col is None else int(gate_col), _ptr(gate_out), _ptr(ssq), int(n_partials), int(d),
+                               float(eps), _ptr(norm_out), _stream()), "route")
 
 
-def expert_gemm(a, w, out, act=None, offsets=None, pairs=None, a_div=1, mfma=True, gated=None):
+def expert_gemm(a, w, out, act=None, offsets=None, pairs=None, a_div=1, mfma=True, gated=None, row_in=None, row_out=None):
     """``out[p] = act(w[e] @ a[p // a_div])`` for every pair p of expert e's run (``offsets``, ``pairs`` of ``route``);
     without them ``w`` is one expert [1, N, K] that takes every row of ``a`` in its own order. ``w`` [E, N, K];
     ``out`` [pairs, N] in bfloat16 or float32. ``gated = (activation, limit, shift)``: the rows of every ``w[e]`` are
     gate and up rows in turns (2n: gate n, 2n + 1: up n) and ``out`` [pairs, N / 2] = act(min(gate, limit)) *
     (clamp(up, -limit, limit) + shift) (``limit`` None or 0: unbounded); ``act`` is then None. ``offsets`` may run on
-    behind the E experts of ``w`` (experts without a product of their own): their pairs are left alone."""
+    behind the E experts of ``w`` (experts without a product of their own): their pairs are left alone. ``row_in`` /
+    ``row_out`` (float32, one number per row of ``out``): a factor on the row's input (in front of the activation) / on
+    its output."""
     _dev(a, "a", contiguous=False); _dev(w, "w", a.dtype); _dev(out, "out", contiguous=False)
     n_out = w.shape[1] // 2 if gated is not None and w.dim() == 3 else (w.shape[1] if w.dim() == 3 else -1)
     if w.dim() != 3 or a.dim() != 2 or a.stride(1) != 1 or out.stride(1) != 1 or a.shape[1] != w.shape[2] or out.shape[1] != n_out:
@@ -825,31 +887,44 @@ def expert_gemm(a, w, out, act=None, offsets=None, pairs=None, a_div=1, mfma=Tru
             raise KernelError(f"expert_gemm: {offsets.numel()} offsets, {pairs.numel()} pairs, {a.shape[0]} rows x {a_div}")
     elif E != 1 or a.shape[0] != n_rows or a_div != 1:
         raise KernelError("expert_gemm: without runs one expert takes every row")
+    for f in (row_in, row_out):
+        if f is not None:
+            _dev(f, "row factors", torch.float32)
+            if f.numel() != n_rows:
+                raise KernelError(f"expert_gemm: {f.numel()} factors for {n_rows} rows")
     if act not in EXPERT_ACTIVATIONS:
         raise KernelError(f"expert_gemm: activation {act!r} is not built ({sorted(k for k in EXPERT_ACTIVATIONS if k)})")
     _check(library().gl3_expert_gemm(_ptr(a), _code(a, "a"), a.stride(0), int(a_div), _ptr(w), _code(w, "w"), E, N, K,
                                      _ptr(offsets), _ptr(pairs), n_rows, _ptr(out), _code(out, "out"), out.stride(0),
-                                     EXPERT_ACTIVATIONS[act], int(bool(mfma)), gate_act, limit, shift, _stream()), "expert_gemm")
+                                     EXPERT_ACTIVATIONS[act], int(bool(mfma)), gate_act, limit, shift, _ptr(row_in),
+                                     _ptr(row_out), _stream()), "expert_gemm")
 
 
-def route_combine(y, wts, out, accumulate=False, identity=None):
+def route_combine(y, wts, out, accumulate=False, identity=None, ssq=None, next_weight=None, xg=None):
     """``out[t]`` (+)= sum over j of ``wts[t, j] * y[t * top + j]``; y [T top, d] float32, out [T, d] float32.
     ``identity = (idx [T, top] int32, n_real, h [T, d])``: a pair whose expert number is ``n_real`` or more stands for
-    the token's input row ``h[t]`` itself."""
+    the token's input row ``h[t]`` itself. ``ssq`` [1, 64] with ``next_weight`` float32 [d] and ``xg`` bfloat16 [T, d] (at
+    most 64 tokens, with ``accumulate``): also the completed rows' sums of squares and the rows times the next norm's
+    weight, for a norm that is folded into the product that follows."""
     _dev(y, "y", torch.float32); _dev(wts, "wts", torch.float32); _dev(out, "out", torch.float32)
     T, top = wts.shape
     if y.dim() != 2 or y.shape[0] != T * top or out.shape != (T, y.shape[1]):
         raise KernelError(f"route_combine: y {tuple(y.shape)}, wts {tuple(wts.shape)}, out {tuple(out.shape)}")
     idx = h = None
     n_real = 0
+    if ssq is not None:
+        _dev(ssq, "ssq", torch.float32)
+        if T > 64 or not accumulate or identity is not None or ssq.numel() < 64 or xg is None or not xg.is_contiguous():
+            raise KernelError("route_combine: what a folded norm reads goes with at most 64 rows that are added to")
+    _check_next(next_weight, xg, T, y.shape[1], "route_combine")
     if identity is not None:
         idx, n_real, h = identity
         _dev(idx, "idx", torch.int32); _dev(h, "h")
         if idx.shape != wts.shape or h.shape != out.shape:
             raise KernelError(f"route_combine: choices {tuple(idx.shape)}, input rows {tuple(h.shape)}")
     _check(library().gl3_route_combine(_ptr(y), _ptr(wts), T, top, y.shape[1], _ptr(out), int(bool(accumulate)), _ptr(idx),
-                                       int(n_real), _ptr(h), _code(h, "h") if h is not None else 0, _stream()),
-           "route_combine")
+                                       int(n_real), _ptr(h), _code(h, "h") if h is not None else 0, _ptr(ssq),
+                                       _ptr(next_weight), _ptr(xg), _stream()), "route_combine")
 
 
 def streams_step(rows, S, y=None, mix=None, out_w=None, in_w=None, norm_w=None, eps=0.0, h=None):
@@ -1633,6 +1708,9 @@ def qkv_rope_cache(a, ssq, n_partials, eps, w_qkv, q_out, positions, seq_of_toke
 
 
 # ------------------------------------------------------------------ bfloat16 attention of a decode step
+ATTENTION_HEAD_SIZES = (32, 64, 96, 128)       # what the matrix-core attention kernels are built for (keys and values alike)
+
+
 def attention_decode_fits(head_dim, n_heads, n_kv, page_size):
     return bool(library().gl3_attention_decode_supports(head_dim, page_size)) and n_heads % n_kv == 0
 
@@ -1655,8 +1733,8 @@ def decode_splits(n_tokens, n_heads, n_kv, kv_len, head_dim=64):
 
 def attention_decode(q, k_cache, v_cache, positions, seq_of_token, block_table, out, n_heads, n_kv, head_dim,
                      page_size, window, scale, n_splits, part_o=None, part_ml=None, slopes=None, sink=None, keep_first=0,
-                     chunk=0, n_v_heads=None):
-    """``slopes`` (float32 [H]): score - slopes[h] * distance; ``sink``: the score of a key without a value that every
+                     chunk=0, n_v_heads=None, rule=None):
+    """``rule``: a ``ScoreRule``; ``slopes`` (float32 [H]): score - slopes[h] * distance; ``sink``: the score of a key without a value that every
     query sees (None: none); ``keep_first``: with a window, the sequence's first keys that stay visible; ``chunk`` and
     ``n_v_heads`` as in ``attention_generic``. One token per sequence. ``part_o`` [T, H, splits, hs] and ``part_ml`` [T, H, splits, 2] float32
     are needed when ``n_splits`` > 1 (contiguous, adjacent is not required). ``seq_of_token`` None: token t's
@@ -1690,7 +1768,7 @@ def attention_decode(q, k_cache, v_cache, positions, seq_of_token, block_table, 
         block_table.shape[1], _ptr(part_o), _ptr(part_ml), floats, _ptr(out), out.stride(0), T, n_heads, n_kv,
         head_dim, page_size, int(window or 0), float(scale), n_splits, _slopes(slopes, n_heads, "attention_decode"),
         has_sink, sink_value, int(keep_first or 0) if window else 0, int(chunk or 0), n_kv // n_v, sinks,
-        _stream()), "attention_decode")
+        *_rule(rule, T, n_heads * head_dim, q.dtype, "attention_decode"), _stream()), "attention_decode")
 
 
 # ------------------------------------------------------------------ bfloat16 product for many rows
@@ -1776,8 +1854,8 @@ def attention_prefill_fits(head_dim, n_heads, n_kv, page_size):
 
 def attention_prefill(q, k_cache, v_cache, cu_seqlens, kv_before, block_table, out, max_q_len, n_heads, n_kv,
                       head_dim, page_size, window, scale, seq_rows=None, wide_from=0, slopes=None, sink=None, keep_first=0,
-                      chunk=0, n_v_heads=None):
-    """``slopes`` (float32 [H]): score - slopes[h] * distance; ``sink``: the score of a key without a value that every
+                      chunk=0, n_v_heads=None, rule=None):
+    """``rule``: a ``ScoreRule``; ``slopes`` (float32 [H]): score - slopes[h] * distance; ``sink``: the score of a key without a value that every
     query sees (None: none); ``chunk`` and ``n_v_heads`` as in ``attention_generic``. Any number of tokens per sequence; ``cu_seqlens`` [B+1] and ``kv_before`` [B] say which tokens
     of the packed ``q`` belong to which sequence and where they sit in it. ``seq_rows`` [B] (optional)
     names each sequence's row of ``block_table``; without it sequence b reads row b. ``wide_from``: from
@@ -1811,7 +1889,7 @@ def attention_prefill(q, k_cache, v_cache, cu_seqlens, kv_before, block_table, o
         _ptr(seq_rows), block_table.shape[1], _ptr(out), out.stride(0), B, int(max_q_len), n_heads, n_kv, head_dim,
         page_size, int(window or 0), float(scale), int(wide_from), _slopes(slopes, n_heads, "attention_prefill"),
         has_sink, sink_value, int(keep_first or 0) if window else 0, int(chunk or 0), n_kv // n_v, sinks,
-        _stream()), "attention_prefill")
+        *_rule(rule, T, n_heads * head_dim, q.dtype, "attention_prefill"), _stream()), "attention_prefill")
 
 
 # ------------------------------------------------------------------ host to device without tensor objects

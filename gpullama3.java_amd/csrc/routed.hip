@@ -14,15 +14,34 @@
 // over the chosen logits alone -> wts [T][top]. One thread a token.
 // With `scores` set the rule is another: s = softmax over all E logits; the choice goes by s + correction[e]
 // (correction may be null), the weights are the chosen s themselves divided by their sum plus sum_eps.
+// A third rule (scores 2): s = sigmoid of every logit, the largest are chosen, their weights are their s as they are.
+//
+// RouteExtras: rows of logits of `ld` floats. `in_wts` (not null): a pair's weight multiplies its expert's INPUT: it is
+// written here and the weight of its output (wts) is 1. `gate_col` (not negative): the output of the expert that
+// every token passes is multiplied by sigmoid(logits[gate_col]), which goes to that expert's pair in wts, or to gate_out
+// [T] where it has no pair. ssq (not null): the rows that the experts will multiply are not normed yet; [n_partials][64]
+// partial sums of squares of the residual rows (at most 64 of them), from which 1 / sqrt(sum / d + eps) is made and
+// multiplied into in_wts (for a pair whose weight is 1 too) and handed out as norm_out [T].
+struct RouteExtras {
+  int ld;
+  float* in_wts;
+  int gate_col;
+  float* gate_out;
+  const float* ssq;
+  int n_partials, d;
+  float eps;
+  float* norm_out;
+};
 __device__ __forceinline__ void route_choose(const float* __restrict__ logits, int t, int E, int top, int* idx,
                                              float* __restrict__ wts, int always, int scores,
-                                             const float* __restrict__ correction, float sum_eps) {
-  const float* z = logits + (long)t * E;
+                                             const float* __restrict__ correction, float sum_eps, const RouteExtras& x,
+                                             float inv_rms) {
+  const float* z = logits + (long)t * x.ld;
   const int stride = top + (always >= 0 ? 1 : 0);
   int chosen[ROUTE_MAX_TOP];
   float val[ROUTE_MAX_TOP];
   float z_max = -INFINITY, z_sum = 1.f;
-  if (scores) {
+  if (scores == 1) {
     for (int e = 0; e < E; ++e) z_max = fmaxf(z_max, z[e]);
     z_sum = 0.f;
     for (int e = 0; e < E; ++e) z_sum += expf(z[e] - z_max);
@@ -33,8 +52,8 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, i
     for (int e = 0; e < E; ++e) {
       bool taken = false;
       for (int i = 0; i < j; ++i) taken |= chosen[i] == e;
-      const float sc = scores ? expf(z[e] - z_max) / z_sum : z[e];
-      const float v = (scores && correction) ? sc + correction[e] : sc;
+      const float sc = scores == 1 ? expf(z[e] - z_max) / z_sum : z[e];      // (a sigmoid keeps the logits' order)
+      const float v = (scores == 1 && correction) ? sc + correction[e] : sc;
       if (!taken && (best < 0 || v > bv)) {
         best = e;
         bv = v;
@@ -45,7 +64,10 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, i
     val[j] = bs;
   }
   float sum = 0.f;
-  if (scores) {
+  if (scores == 2) {
+    for (int j = 0; j < top; ++j) val[j] = 1.0f / (1.0f + expf(-val[j]));
+    sum = 1.f;
+  } else if (scores == 1) {
     for (int j = 0; j < top; ++j) sum += val[j];
     sum += sum_eps;
   } else {
@@ -57,19 +79,25 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, i
   }
   for (int j = 0; j < top; ++j) {
     idx[(long)t * stride + j] = chosen[j];
-    wts[(long)t * stride + j] = val[j] / sum;
+    const float w = val[j] / sum;
+    wts[(long)t * stride + j] = x.in_wts ? 1.0f : w;
+    if (x.in_wts) x.in_wts[(long)t * stride + j] = w * inv_rms;
   }
+  const float gate = x.gate_col >= 0 ? 1.0f / (1.0f + expf(-z[x.gate_col])) : 1.0f;
   if (always >= 0) {                     // one more pair per token: the expert that every token passes, with weight 1
     idx[(long)t * stride + top] = always;
-    wts[(long)t * stride + top] = 1.0f;
+    wts[(long)t * stride + top] = gate;
+    if (x.in_wts) x.in_wts[(long)t * stride + top] = inv_rms;
   }
+  if (x.gate_out) x.gate_out[t] = gate;
+  if (x.norm_out) x.norm_out[t] = inv_rms;
 }
 
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ logits, int T, int E, int top,
                                                          int* __restrict__ idx, float* __restrict__ wts, int always, int scores,
-                                                         const float* __restrict__ correction, float sum_eps) {
+                                                         const float* __restrict__ correction, float sum_eps, RouteExtras x) {
   const int t = blockIdx.x * 64 + threadIdx.x;
-  if (t < T) route_choose(logits, t, E, top, idx, wts, always, scores, correction, sum_eps);
+  if (t < T) route_choose(logits, t, E, top, idx, wts, always, scores, correction, sum_eps, x, 1.0f);
 }
 
 // ----------------------------------------------------------------- pairs ordered by expert
@@ -107,8 +135,21 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(const int* __restrict_
 __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict__ logits, int T, int E, int top,
                                                           int* idx, float* __restrict__ wts,
                                                           int* __restrict__ offsets, int* __restrict__ sorted, int always,
-                                                          int scores, const float* __restrict__ correction, float sum_eps) {
-  if ((int)threadIdx.x < T) route_choose(logits, threadIdx.x, E, top, idx, wts, always, scores, correction, sum_eps);
+                                                          int scores, const float* __restrict__ correction, float sum_eps,
+                                                          RouteExtras x) {
+  __shared__ float inv_rms[64];
+  if (x.ssq) {                              // (the same for all threads) a wave a row adds up its partial sums
+    for (int t = threadIdx.x >> 6; t < T; t += blockDim.x >> 6) {
+      float s = 0.f;
+      for (int i = threadIdx.x & 63; i < x.n_partials; i += 64) s += x.ssq[(long)i * 64 + t];
+      s = wave_sum(s);
+      if ((threadIdx.x & 63) == 0) inv_rms[t] = 1.0f / sqrtf(s / (float)x.d + x.eps);
+    }
+    __syncthreads();
+  }
+  if ((int)threadIdx.x < T)
+    route_choose(logits, threadIdx.x, E, top, idx, wts, always, scores, correction, sum_eps, x,
+                 x.ssq ? inv_rms[threadIdx.x] : 1.0f);
   __threadfence_block();
   __syncthreads();
   const int more = always >= 0 ? 1 : 0;
@@ -118,21 +159,29 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
 // `always` (-1: none): the number E of one more expert behind the router's, which every token passes with weight 1; idx
 // and wts then have top + 1 entries a token, offsets E + 2.
 extern "C" int gl3_route(const float* logits, int n_tokens, int E, int top, int* idx, float* wts, int* offsets, int* sorted,
-                         int always, int scores, const float* correction, float sum_eps, hipStream_t stream) {
+                         int always, int scores, const float* correction, float sum_eps, int ld, float* in_wts, int gate_col,
+                         float* gate_out, const float* ssq, int n_partials, int d, float eps, float* norm_out,
+                         hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(logits && idx && wts && offsets && sorted, "gl3_route: null argument");
   const int more = always >= 0 ? 1 : 0;
   GL3_REQUIRE(n_tokens > 0 && E >= 1 && E + more <= ROUTE_MAX_EXPERTS && top >= 1 && top <= ROUTE_MAX_TOP && top <= E,
               "gl3_route: the %d largest of %d experts (at most %d of %d)", top, E, ROUTE_MAX_TOP, ROUTE_MAX_EXPERTS);
   GL3_REQUIRE(always < 0 || always == E, "gl3_route: the expert that every token passes is number %d, not %d", E, always);
+  GL3_REQUIRE(scores >= 0 && scores <= 2 && ld >= E && gate_col < ld, "gl3_route: rule %d, rows of %d for %d experts, gate in column %d",
+              scores, ld, E, gate_col);
+  GL3_REQUIRE(!gate_out || gate_col >= 0, "gl3_route: a gate to hand out without a column of logits for it");
+  GL3_REQUIRE(!ssq || (n_tokens <= 64 && n_partials > 0 && d > 0 && in_wts),
+              "gl3_route: a norm carried by the pairs' weights takes at most 64 tokens and weights on the experts' inputs");
+  const RouteExtras x{ld, in_wts, gate_col, gate_out, ssq, n_partials, d, eps, norm_out};
   if (n_tokens <= 64) {
     route_few_kernel<<<dim3(1), dim3(1024), 0, stream>>>(logits, n_tokens, E, top, idx, wts, offsets, sorted, always, scores,
-                                                         correction, sum_eps);
+                                                         correction, sum_eps, x);
     GL3_LAUNCH_CHECK();
     return 0;
   }
   route_topk_kernel<<<dim3((n_tokens + 63) / 64), dim3(64), 0, stream>>>(logits, n_tokens, E, top, idx, wts, always, scores,
-                                                                                 correction, sum_eps);
+                                                                                 correction, sum_eps, x);
   GL3_LAUNCH_CHECK();
   route_sort_kernel<<<dim3(1), dim3(1024), 0, stream>>>(idx, n_tokens * (top + more), E + more, offsets, sorted);
   GL3_LAUNCH_CHECK();
@@ -154,15 +203,23 @@ __device__ __forceinline__ float gl3_expert_act(float v, int act) {
 // holds column c of the sums finds its partner's in the lane beside it; the even one writes column c / 2 of the
 // output: act(gate) * (up + shift), both bounded by `limit` first where it is positive (gl3_gated). Every lane of a
 // wave must come here (the partner's value travels from lane to lane); `ok` says whether this lane's element exists.
+// RowFactors: numbers per row (pair) that may be null: `in` multiplies the row's input (its sums, in front of the
+// activation), `out` its output (behind it).
+struct RowFactors {
+  const float* in;
+  const float* out;
+};
 template <typename TO>
 __device__ __forceinline__ void expert_store(TO* __restrict__ out, long ldo, int row, int n, bool ok, float v, int act,
-                                             int gate_act, float limit, float shift) {
+                                             int gate_act, float limit, float shift, const RowFactors& f) {
+  if (f.in) v *= ok ? f.in[row] : 0.f;
+  const float after = f.out && ok ? f.out[row] : 1.f;
   if (gate_act < 0) {
-    if (ok) out[(long)row * ldo + n] = from_f32<TO>(gl3_expert_act(v, act));
+    if (ok) out[(long)row * ldo + n] = from_f32<TO>(gl3_expert_act(v, act) * after);
     return;
   }
   const float up = __shfl_xor(v, 1, 64);
-  if (ok && !(n & 1)) out[(long)row * ldo + (n >> 1)] = from_f32<TO>(gl3_gated<false>(v, up, gate_act, limit, shift));
+  if (ok && !(n & 1)) out[(long)row * ldo + (n >> 1)] = from_f32<TO>(gl3_gated<false>(v, up, gate_act, limit, shift) * after);
 }
 
 __device__ __forceinline__ bool expert_tile(const int* offsets, int E, int n_rows, int TM, int tile, int* e_out, int* lo_out,
@@ -196,7 +253,7 @@ __global__ __launch_bounds__(256) void expert_gemm_generic_kernel(const TA* __re
                                                                    const int* __restrict__ offsets,
                                                                    const int* __restrict__ sorted, int E, int n_rows,
                                                                    TO* __restrict__ out, long ldo, int act, int gate_act, float limit,
-                                                                   float shift) {
+                                                                   float shift, RowFactors rf) {
   __shared__ float sa[EG_TM][EG_TK + 1];
   __shared__ float sw[EG_TN][EG_TK + 1];
   __shared__ int rows[EG_TM];
@@ -230,7 +287,7 @@ __global__ __launch_bounds__(256) void expert_gemm_generic_kernel(const TA* __re
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int n = n0 + cg + 16 * j;
-    expert_store<TO>(out, ldo, rows[r], n, rows[r] >= 0 && n < N, acc[j], act, gate_act, limit, shift);
+    expert_store<TO>(out, ldo, rows[r], n, rows[r] >= 0 && n < N, acc[j], act, gate_act, limit, shift, rf);
   }
 }
 
@@ -247,7 +304,7 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(const bf16_t* __r
                                                                 const int* __restrict__ offsets,
                                                                 const int* __restrict__ sorted, int E, int n_rows,
                                                                 TO* __restrict__ out, long ldo, int act, int gate_act, float limit,
-                                                                   float shift) {
+                                                                   float shift, RowFactors rf) {
   __shared__ int rows[EM_TM];
   int e, lo, hi;
   if (!expert_tile(offsets, E, n_rows, EM_TM, blockIdx.x, &e, &lo, &hi)) return;
@@ -289,7 +346,7 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(const bf16_t* __r
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int row = rows[g * 16 + (lane >> 4) * 4 + i];
-      expert_store<TO>(out, ldo, row, nc, row >= 0 && nc < N, acc[g][i], act, gate_act, limit, shift);
+      expert_store<TO>(out, ldo, row, nc, row >= 0 && nc < N, acc[g][i], act, gate_act, limit, shift, rf);
     }
   }
 }
@@ -308,7 +365,7 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
                                                                         const int* __restrict__ offsets,
                                                                         const int* __restrict__ sorted, int E, int n_rows,
                                                                         TO* __restrict__ out, long ldo, int act, int gate_act, float limit,
-                                                                   float shift) {
+                                                                   float shift, RowFactors rf) {
   constexpr int TM = 16 * G;
   __shared__ int rows[TM];
   __shared__ float part[EF_WAVES][TM][EF_TN + 1];
@@ -375,7 +432,7 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
 #pragma unroll
     for (int w = 0; w < EF_WAVES; ++w) sum += part[w][r][c];
     const int nc = blockIdx.y * EF_TN + c;
-    expert_store<TO>(out, ldo, rows[r], nc, in && nc < N, sum, act, gate_act, limit, shift);
+    expert_store<TO>(out, ldo, rows[r], nc, in && nc < N, sum, act, gate_act, limit, shift, rf);
   }
 }
 
@@ -396,7 +453,7 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
                                                                  const int* __restrict__ offsets,
                                                                  const int* __restrict__ sorted, int E, int n_rows,
                                                                  TO* __restrict__ out, long ldo, int act, int gate_act, float limit,
-                                                                   float shift) {
+                                                                   float shift, RowFactors rf) {
   constexpr int NT = 512, NA = ET_BM * 8 / NT, NWC = ET_BN * 8 / NT;
   __shared__ __attribute__((aligned(16))) bf16_t As[2][ET_BM][ET_LD];
   __shared__ __attribute__((aligned(16))) bf16_t Ws[2][ET_BN][ET_LD];
@@ -481,14 +538,16 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
 #pragma unroll
     for (int tn = 0; tn < 2; ++tn) {
       const int n = n0 + wn * 64 + tn * 32 + lr;
-      expert_store<TO>(out, ldo, row, n, row >= 0 && n < N, acc[tn][v], act, gate_act, limit, shift);
+      expert_store<TO>(out, ldo, row, n, row >= 0 && n < N, acc[tn][v], act, gate_act, limit, shift, rf);
     }
   }
 }
 
 extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, const void* W, int w_dtype, int E, int N, int K,
                                const int* offsets, const int* sorted, int n_rows, void* out, int out_dtype, long ldo, int act,
-                               int use_mfma, int gate_act, float limit, float shift, hipStream_t stream) {
+                               int use_mfma, int gate_act, float limit, float shift, const float* row_in, const float* row_out,
+                               hipStream_t stream) {
+  const RowFactors rf{row_in, row_out};
   if (n_rows == 0) return 0;
   GL3_REQUIRE(A && W && out && n_rows > 0 && E >= 1 && N > 0 && K > 0 && a_div >= 1 && lda >= K &&
                   ldo >= (gate_act >= 0 ? N / 2 : N),
@@ -507,10 +566,10 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
     const dim3 grid((n_rows + ET_BM - 1) / ET_BM + (offsets ? E : 0), (N + ET_BN - 1) / ET_BN), block(512);
     if (out_dtype == GL3_BF16)
       expert_gemm_tiled_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
-                                                                   sorted, E, n_rows, (bf16_t*)out, ldo, act, gate_act, limit, shift);
+                                                                   sorted, E, n_rows, (bf16_t*)out, ldo, act, gate_act, limit, shift, rf);
     else
       expert_gemm_tiled_kernel<float><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
-                                                                  sorted, E, n_rows, (float*)out, ldo, act, gate_act, limit, shift);
+                                                                  sorted, E, n_rows, (float*)out, ldo, act, gate_act, limit, shift, rf);
     GL3_LAUNCH_CHECK();
     return 0;
   }
@@ -522,7 +581,7 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
     const dim3 grid((n_rows + 16 * G - 1) / (16 * G) + (offsets ? E : 0), (N + EF_TN - 1) / EF_TN), block(EF_WAVES * 64);
 #define EF_LAUNCH(TO, G)                                                                                                \
   expert_gemm_few_kernel<TO, G><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets, \
-                                                            sorted, E, n_rows, (TO*)out, ldo, act, gate_act, limit, shift)
+                                                            sorted, E, n_rows, (TO*)out, ldo, act, gate_act, limit, shift, rf)
     if (out_dtype == GL3_BF16) {
       if (G == 1) EF_LAUNCH(bf16_t, 1); else if (G == 2) EF_LAUNCH(bf16_t, 2); else EF_LAUNCH(bf16_t, 4);
     } else {
@@ -537,10 +596,10 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
     const dim3 grid((n_rows + EM_TM - 1) / EM_TM + (offsets ? E : 0), (N + EM_TN - 1) / EM_TN), block(256);
     if (out_dtype == GL3_BF16)
       expert_gemm_mfma_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
-                                                                  sorted, E, n_rows, (bf16_t*)out, ldo, act, gate_act, limit, shift);
+                                                                  sorted, E, n_rows, (bf16_t*)out, ldo, act, gate_act, limit, shift, rf);
     else if (out_dtype == GL3_F32)
       expert_gemm_mfma_kernel<float><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
-                                                                 sorted, E, n_rows, (float*)out, ldo, act, gate_act, limit, shift);
+                                                                 sorted, E, n_rows, (float*)out, ldo, act, gate_act, limit, shift, rf);
     else GL3_REQUIRE(false, "gl3_expert_gemm: unknown output dtype %d", out_dtype);
     GL3_LAUNCH_CHECK();
     return 0;
@@ -548,7 +607,7 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
   const dim3 grid((n_rows + EG_TM - 1) / EG_TM + (offsets ? E : 0), (N + EG_TN - 1) / EG_TN), block(256);
 #define EG_LAUNCH(TA, TW, TO)                                                                                          \
   expert_gemm_generic_kernel<TA, TW, TO><<<grid, block, 0, stream>>>((const TA*)A, lda, a_div, (const TW*)W, N, K, offsets, \
-                                                                     sorted, E, n_rows, (TO*)out, ldo, act, gate_act, limit, shift)
+                                                                     sorted, E, n_rows, (TO*)out, ldo, act, gate_act, limit, shift, rf)
   if (a_dtype == GL3_F32 && w_dtype == GL3_F32 && out_dtype == GL3_F32) EG_LAUNCH(float, float, float);
   else if (a_dtype == GL3_BF16 && w_dtype == GL3_BF16 && out_dtype == GL3_BF16) EG_LAUNCH(bf16_t, bf16_t, bf16_t);
   else if (a_dtype == GL3_BF16 && w_dtype == GL3_BF16 && out_dtype == GL3_F32) EG_LAUNCH(bf16_t, bf16_t, float);
@@ -578,13 +637,44 @@ __global__ void route_combine_kernel(const float* __restrict__ y, const float* _
   out[i] = s;
 }
 
+// The same, a block a row, for a step of few rows whose completed row a norm folded into the next product will read: also
+// ssq[t] = the row's sum of squares and xg[t] = bfloat16(next_weight * row).
+__global__ __launch_bounds__(1024) void route_combine_norm_kernel(const float* __restrict__ y, const float* __restrict__ wts,
+                                                                   int top, int d, float* __restrict__ out,
+                                                                   float* __restrict__ ssq,
+                                                                   const float* __restrict__ next_weight,
+                                                                   bf16_t* __restrict__ xg) {
+  __shared__ float scratch[16];
+  const long t = blockIdx.x;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < d; c += blockDim.x) {
+    float s = out[t * d + c];
+    for (int j = 0; j < top; ++j) s = fmaf(wts[t * top + j], y[(t * top + j) * d + c], s);
+    out[t * d + c] = s;
+    xg[t * d + c] = static_cast<bf16_t>(next_weight[c] * s);
+    ss += s * s;
+  }
+  ss = block_sum(ss, scratch);
+  if (threadIdx.x == 0) ssq[t] = ss;
+}
+
 extern "C" int gl3_route_combine(const float* y, const float* wts, int n_tokens, int top, int d, float* out, int accumulate,
-                                 const int* idx, int n_real, const void* h, int h_dtype, hipStream_t stream) {
+                                 const int* idx, int n_real, const void* h, int h_dtype, float* ssq,
+                                 const float* next_weight, void* xg, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(y && wts && out && n_tokens > 0 && top >= 1 && d > 0, "gl3_route_combine: bad arguments");
   GL3_REQUIRE((idx == nullptr) == (h == nullptr), "gl3_route_combine: identity experts need the choices and the input rows");
   const long n = (long)n_tokens * d;
   GL3_REQUIRE((n + 255) / 256 < (1L << 31), "gl3_route_combine: too many elements");
+  GL3_REQUIRE((ssq == nullptr) == (next_weight == nullptr) && (ssq == nullptr) == (xg == nullptr) &&
+                  (!ssq || (n_tokens <= 64 && accumulate && !idx)),
+              "gl3_route_combine: what a folded norm reads comes together, for at most 64 rows that are added to");
+  if (ssq) {
+    const int threads = d >= 1024 ? 1024 : ((d + 63) / 64) * 64;
+    route_combine_norm_kernel<<<dim3(n_tokens), dim3(threads), 0, stream>>>(y, wts, top, d, out, ssq, next_weight, (bf16_t*)xg);
+    GL3_LAUNCH_CHECK();
+    return 0;
+  }
   if (h && h_dtype == GL3_BF16)
     route_combine_kernel<bf16_t><<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream>>>(y, wts, top, d, out, accumulate, n,
                                                                                             idx, n_real, (const bf16_t*)h);

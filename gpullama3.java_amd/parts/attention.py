@@ -22,7 +22,13 @@ stored head by head as [map 1, map 2], and the cache keeps twice the key heads b
 without keys and values of its own (no ``k`` among its names) that only ever reads another entry's; a learned sink per
 query head (a stored [n_heads] vector named ``sink``, on every kernel that knows a sink); and values that are the keys
 as projected (``values_are_keys``: no value projection; the key rows stand twice in the stacked product, once to be
-normed and turned, once to be cached as they are).
+normed and turned, once to be cached as they are). Also on that path, in every kernel that such a step may take
+(``lib.ScoreRule``): a soft cap on the scores in front of the distance bias (``score_softcap``), queries that count more
+the further on they stand (``query_temperature``), a gate per element of the heads' outputs (a matrix named ``gate``, more
+rows of the stacked product; the attention kernel applies it where it writes its output). And values blended across
+layers (``value_mix``): the first such layer's stacked rows stay where they are for the rest of the step, and the later
+ones' cache write reads them beside its own. Where such an attention has no rotation, a bfloat16 engine stores keys and
+values in one size that the matrix-core kernels are built for, padded with zeros.
 """
 from __future__ import annotations
 
@@ -70,9 +76,30 @@ class GQAAttention:
         self.general = bool(self.value_position_spec is not None or self.gated
                             or (spec.position is not None and self.vd != self.hs) or self.qk_norm_eps is not None
                             or self.diff is not None or self.reads_only or self.values_are_keys)
+        # (a rule on scores and outputs and values blended across layers: the same path)
+        self.cap = getattr(spec, "score_softcap", None)
+        self.temperature = getattr(spec, "query_temperature", None)
+        self.mix = getattr(spec, "value_mix", None)
+        self.gated_elements = "gate" in spec.names
+        ruled = self.cap is not None or self.temperature is not None or self.gated_elements
+        if ruled or self.mix is not None:
+            if self.diff is not None or self.reads_only or self.values_are_keys or self.value_position_spec is not None:
+                raise ValueError("an attention with a rule on its scores and outputs, or with values blended across layers, "
+                                 "has one score map and plain values of its own")
+            if self.gated and self.gated_elements:
+                raise ValueError("an attention has a gate per head or a gate per element, not both")
+            self.general = True
+        self.ruled = ruled
         if spec.position is None or self.general:
             # (a rotation touches a head's first elements only: zeros behind them stay zeros)
             self.hs, self.vd = -(-self.hs // 16) * 16, -(-self.vd // 16) * 16
+        # what turns or norms heads, or gates them as a whole, goes through the kernel that does all of these
+        self.turns = bool(spec.position is not None or self.value_position_spec is not None or self.gated
+                          or self.qk_norm_eps is not None)
+        if self.general and (ruled or self.mix is not None) and not self.turns and dtype == torch.bfloat16:
+            one = [n for n in K.ATTENTION_HEAD_SIZES if n >= max(self.hs, self.vd)]
+            if one:
+                self.hs = self.vd = one[0]
         self.window = spec.window
         self.keep_first = int(getattr(spec, "keep_first", 0) or 0) if spec.window else 0
         self.out_mult = float(getattr(spec, "out_mult", 1.0))
@@ -84,7 +111,7 @@ class GQAAttention:
         self.device = device
         self.out_scale_name = getattr(spec, "out_scale_name", None)
         self.out_scale = None
-        self.scale = spec.scale if spec.scale is not None else 1.0 / math.sqrt(self.hs)
+        self.scale = spec.scale if spec.scale is not None else 1.0 / math.sqrt(self.hs_stored)
         self.position = build_part("position", spec.position, device=device) if spec.position is not None else None
         self.value_position = (build_part("position", self.value_position_spec, device=device)
                                if self.value_position_spec is not None else None)
@@ -122,6 +149,10 @@ class GQAAttention:
             out[self.out_scale_name] = TensorSpec((d,), "vector", 1.0, 0.1)
         if self.gated:
             out[n["head_gate"]] = TensorSpec((self.H, d))
+        if self.gated_elements:
+            out[n["gate"]] = TensorSpec((self.H * vd, d))
+        if self.mix is not None and not self.mix.first:
+            out[n["v_mix"]] = TensorSpec((), "vector", 0.5, 0.1)
         return out
 
     def load(self, weights):
@@ -182,14 +213,15 @@ class GQAAttention:
         if self.reads_only and self.gated:
             raise ValueError("an attention without keys and values of its own is built without a gate per head")
         kinds = ("q",) if self.reads_only else ("q", "k", "k") if self.values_are_keys else ("q", "k", "v")
-        parts = [weights[n[k]] for k in kinds] + ([weights[n["head_gate"]]] if self.gated else [])
+        kinds += (("head_gate",) if self.gated else ()) + (("gate",) if self.gated_elements else ())
+        parts = [weights[n[k]] for k in kinds]
         dt = parts[0].dtype if all(p.dtype == parts[0].dtype for p in parts) else torch.float32
         rows = sum(p.shape[0] for p in parts)
         pad = torch.zeros((-(-rows // 16) * 16 - rows, self.d), dtype=dt, device=parts[0].device)
         self.w_qkv = torch.cat([p.to(dt) for p in parts] + [pad], dim=0).contiguous()
         lo = 0
         named = set()
-        for k, p in zip(kinds + ("head_gate",), parts):      # the stored names stay addressable as views
+        for k, p in zip(kinds, parts):      # the stored names stay addressable as views
             if k not in named:                                # (key rows that stand twice: the first ones)
                 weights[n[k]] = self.w_qkv[lo:lo + p.shape[0]]
                 named.add(k)
@@ -209,6 +241,8 @@ class GQAAttention:
         if self.diff is not None:
             lq1, lk1, lq2, lk2 = (weights[n[k]].float() for k in ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2"))
             self.diff_lambda = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + float(self.diff.offset)
+        if self.mix is not None and not self.mix.first:
+            self.mix_lambda = float(weights[n["v_mix"]])
         self._load_scales(weights)
         if self._slopes_host is not None:
             self.slopes = torch.tensor(self._slopes_host, dtype=torch.float64).to(torch.float32).to(self.w_qkv.device)
@@ -247,14 +281,29 @@ class GQAAttention:
         T, H, Hq, Kq, Kh, hs, vd = h.shape[0], self.H, self.Hq, self.Kq, self.Kh, self.hs, self.vd
         qn, kn, vn = Hq * hs, Kq * hs, Kh * vd
         w = self.w_qkv if writes else self.w_q_rows
-        qkv = ctx.buffer("qkvg", (T, w.shape[0]), self.dtype)
+        # (the first of the layers that blend their values keeps its rows for the others: a buffer that no other writes)
+        hands_out = self.mix is not None and self.mix.first
+        qkv = ctx.buffer("qkvg_first_values" if hands_out else "qkvg", (T, w.shape[0]), self.dtype)
         ops.linear(h, w, qkv, ops.EPI_STORE, ctx)
         pos, vpos = self.position, self.value_position
         # q, k and v normed and turned in place, k and v into the cache as they come out: one kernel
         qk = (pos.rot_dim, pos.cos, pos.sin) if pos is not None else (0, None, None)
         vr = (vpos.rot_dim, vpos.cos, vpos.sin) if vpos is not None else (0, None, None)
         normed = self.qk_norm_eps is not None
-        if writes:
+        if hands_out:
+            ctx.first_values = (qkv[:, qn + kn:qn + kn + vn], vd, self.vd_stored)
+        blend = None
+        if self.mix is not None and not self.mix.first:
+            other = getattr(ctx, "first_values", None)
+            if other is None or other[2] != self.vd_stored or other[0].shape[1] != Kh * other[1]:
+                raise ValueError("an attention that blends its values finds no earlier layer's values of the same heads and size")
+            blend = (other[0], other[1], self.mix_lambda)
+        if writes and not self.turns:
+            K.kv_write(qkv, qn, qn + kn, ctx.positions, ops._table_rows(ctx), table, k_cache, v_cache, Kh, hs, vd,
+                       k_cache.shape[2], blend=blend)
+        elif blend is not None:
+            raise NotImplementedError("values blended across layers beside a rotation are not built")
+        elif writes:
             K.rotate_heads(qkv, ctx.positions, [(0, Hq, hs) + qk, (qn, Kq, hs) + qk, (qn + kn, Kh, vd) + vr],
                            adjacent=bool(pos.adjacent if pos is not None else vpos is not None and vpos.adjacent),
                            cache=(k_cache, v_cache, ops._table_rows(ctx), table, k_cache.shape[2]),
@@ -269,7 +318,7 @@ class GQAAttention:
         att = ctx.buffer("attn_out", (T, Hq * vd), att_dtype)
         ops.attention(ctx, qkv, k_cache, v_cache, table, att, Hq, Kq, hs, self.window, self.scale, v_head_dim=vd,
                       slopes=self.slopes, sink=self.sink, keep_first=self.keep_first, chunk=self.chunk,
-                      n_v_heads=Kh if self.maps > 1 else None)
+                      n_v_heads=Kh if self.maps > 1 else None, rule=self._score_rule(qkv, qn + kn + vn))
         if self.diff is not None:
             # the two maps' outputs of every head into one: a1 - lambda a2, a unit norm per head, the factor 1 - offset
             both, att = att, ctx.buffer("attn_maps_joined", (T, H * vd), self.dtype)      # (the activations' type again)
@@ -282,6 +331,14 @@ class GQAAttention:
                            adjacent=bool(vpos is not None and vpos.adjacent), back=True,
                            gate=qkv if self.gated else None, gate_col=qn + kn + vn)
         ops.linear(att, self.w_o, x, epilogue, ctx, col_scale=self.out_scale)
+
+    def _score_rule(self, qkv, col):
+        """What the attention kernels do beyond the plain rule; ``col``: where the gate's columns begin."""
+        if not self.ruled:
+            return None
+        t = self.temperature
+        return K.ScoreRule(self.cap, (t.coef, t.every) if t is not None else None,
+                           qkv[:, col:col + self.H * self.vd] if self.gated_elements else None)
 
     def _project_unequal(self, ctx, h, k_cache, v_cache, table, run):
         """Values of another size than the keys: one product over the stacked rows, then keys and values into the
@@ -309,7 +366,7 @@ class _PaddedHeads:
         p, n, w = self.part, self.part.names, self.weights[name]
         heads = {n["q"]: (p.Hq, p.hs_stored, p.hs), n.get("k"): (p.Kq, p.hs_stored, p.hs), n.get("v"): (p.Kh, p.vd_stored, p.vd),
                  n.get("q_bias"): (p.Hq, p.hs_stored, p.hs), n.get("k_bias"): (p.Kq, p.hs_stored, p.hs),
-                 n.get("v_bias"): (p.Kh, p.vd_stored, p.vd)}
+                 n.get("v_bias"): (p.Kh, p.vd_stored, p.vd), n.get("gate"): (p.H, p.vd_stored, p.vd)}
         if name in heads and w.shape[0] == heads[name][0] * heads[name][1]:
             H, d_in, d_out = heads[name]
             out = torch.zeros((H, d_out) + tuple(w.shape[1:]), dtype=w.dtype, device=w.device)

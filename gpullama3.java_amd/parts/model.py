@@ -175,6 +175,7 @@ class DecoderModel:
         x = ctx.buffer("residual", (ctx.n_tokens, self.spec.hidden), torch.float32)
         ctx.ssq = ctx.pending = ctx.next_norm = None   # a context may run more than one forward pass: nothing is left over
         ctx.token_facts, ctx.token_tables = {}, {}
+        ctx.first_values = None         # (the values that later layers of a step blend into theirs, once a layer hands them out)
         ctx.rows_as_input = None        # (the address of rows whose copy in the activations' type a block has left)
         order = [self.blocks[r.layer] for r in self.spec.run_order]
         # the norm that reads the residual rows after entry i of the run order, where the block says which

@@ -482,16 +482,16 @@ def attention_kernel(ctx, dtype, page, n_heads, n_kv, head_dim, scale, v_head_di
 
 
 def attention(ctx, q, k_cache, v_cache, block_table, out, n_heads, n_kv, head_dim, window, scale, v_head_dim=None,
-              slopes=None, sink=None, keep_first=0, chunk=None, n_v_heads=None):
+              slopes=None, sink=None, keep_first=0, chunk=None, n_v_heads=None, rule=None):
     """``v_head_dim``: the values' size (None: the keys'); ``slopes``: float32 [H], a bias of -slopes[h] * distance
     on the scores; ``sink``: the score of a key without a value that every query sees (None: none); ``keep_first``:
     with a window, the sequence's first keys that every later query still sees; ``chunk``: n: a query sees the earlier
     keys of its own run of n positions only; ``n_v_heads``: value heads where several score maps share them
-    (``lib.attention_generic``)."""
+    (``lib.attention_generic``); ``rule``: a ``lib.ScoreRule`` or None."""
     page = k_cache.shape[2]          # keys are [page, kv head, position in page, head_dim]
     extras = dict(slopes=slopes, sink=sink)
     extras["keep_first"] = int(keep_first or 0) if window else 0
-    extras.update(chunk=int(chunk or 0), n_v_heads=n_v_heads)
+    extras.update(chunk=int(chunk or 0), n_v_heads=n_v_heads, rule=rule)
     kernel = attention_kernel(ctx, q.dtype, page, n_heads, n_kv, head_dim, scale, v_head_dim)
     if kernel == "decode":
         T = q.shape[0]
