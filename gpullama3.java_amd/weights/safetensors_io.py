@@ -132,5 +132,5 @@ def write_safetensors(path, tensors, metadata=None):
             t = make().contiguous()
             if tuple(t.shape) != tuple(shape) or t.dtype != dtype:
                 raise ValueError(f"{name}: made {tuple(t.shape)} {t.dtype}, declared {shape} {dtype}")
-            f.write(t.view(torch.uint8).numpy().tobytes() if t.numel() else b"")
+            f.write(t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")
     os.replace(tmp, path)
