@@ -35,7 +35,11 @@ in three quarters of its feed-forward, 2.25 times its feed-forward weights).
 layers in turns of four: a lightning attention, an attention over cached latents, a lightning attention, a windowed
 attention with learned sinks whose values are its keys; the first layer's feed-forward is the shape's own, every other
 layer has 8 gated experts of a quarter of that size and 2 identity experts, two a token, beside a shared expert).
-``--beside nolatar`` puts a Nolatar model of the same sizes beside it instead of the Llama layers.
+``--arch lusalix`` does the same for a Lusalix model (in every layer an attention without a rotation: the shape's heads, a
+temperature on the queries, a soft cap, a distance bias, a window, a gate per element, values blended with the first
+layer's; 8 gated experts of a quarter of the shape's feed-forward size, two a token, beside a shared expert).
+``--beside nolatar`` (or any of the others) puts a model of that design and the same sizes beside it instead of the Llama
+layers.
 """
 import argparse
 import json
@@ -120,10 +124,10 @@ def main():
     ap.add_argument("--points", default="1,64", help="further decode batch sizes, comma-separated")
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--workload", default="decode", choices=["decode", "unequal8"])
-    ap.add_argument("--arch", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex"],
-                    help="melizen, nodupel, nolatar, dotanex: a model of that design with the shape's sizes beside Llama layers of "
+    ap.add_argument("--arch", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex", "lusalix"],
+                    help="melizen, nodupel, nolatar, dotanex, lusalix: a model of that design with the shape's sizes beside Llama layers of "
                          "equal size (a line of its own form)")
-    ap.add_argument("--beside", default="llama", choices=["llama", "melizen", "nodupel", "nolatar"],
+    ap.add_argument("--beside", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex"],
                     help="with --arch: the model of equal size that is measured beside it")
     ap.add_argument("--without", default="", help="names of fast paths to switch off for a comparison on the same machine, "
                     "comma-separated (parts/ops.py: tiled, packed, fused, wide, ...); the line then says so in `config`")
@@ -136,7 +140,7 @@ def main():
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported by this single-GPU library")
         return 2
 
-    if args.arch in ("melizen", "nodupel", "nolatar", "dotanex"):
+    if args.arch != "llama":
         return other_beside_llama(args)
 
     import numpy as np
@@ -414,6 +418,20 @@ def dotanex_config(shape, layers, window=1024, streams=2):
             "max_positions": top, "layers": out}
 
 
+def lusalix_config(shape, layers, window=1024):
+    """A Lusalix model with the sizes of a Llama shape: in every layer an attention with the shape's heads (values of the
+    keys' size), a window, a soft cap of 50 and a temperature that steps every 256 positions, values blended with the first
+    layer's; 8 gated experts of a quarter of the shape's feed-forward size, two a token, and a shared expert of that size."""
+    d, F = shape["hidden_size"], shape["intermediate_size"]
+    H, G, hs = shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
+    mixer = {"heads": H, "kv_heads": G, "dim": hs, "vdim": hs, "scale": hs ** -0.5, "softcap": 50.0,
+             "q_temp": {"coef": 0.1, "every": 256}, "mask": {"size": window}, "v_mix": True}
+    mlp = {"kind": "moe", "router": {"experts": 8, "top": 2}, "expert": {"ff": F // 4}, "shared": {"ff": F // 4}}
+    return {"architecture": "Lusalix", "vocab": shape["vocab_size"], "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+            "max_positions": shape["max_position_embeddings"],
+            "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp} for _ in range(layers)]}
+
+
 def other_beside_llama(args):
     """Prefill of one prompt and decode steps at --batch for a model of another design (--arch) and for Llama layers
     of equal size, one after the other on the same machine."""
@@ -429,7 +447,8 @@ def other_beside_llama(args):
     per_seq = -(-(prompt_len + K + W + 1) // 64) * 64
     short = "bf16" if args.dtype == "bfloat16" else "fp32"
     arch = args.arch
-    makers = {"melizen": melizen_config, "nodupel": nodupel_config, "nolatar": nolatar_config, "dotanex": dotanex_config}
+    makers = {"melizen": melizen_config, "nodupel": nodupel_config, "nolatar": nolatar_config, "dotanex": dotanex_config,
+              "lusalix": lusalix_config}
     beside = "llama" if args.beside == arch else args.beside
     configs = {arch: g.config_from_dict(makers[arch](shape, layers)),
                beside: g.config_from_dict({**shape, "num_hidden_layers": layers} if beside == "llama"

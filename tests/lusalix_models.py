@@ -103,8 +103,9 @@ def tokens(name, seed, n):
 # fraction of the root mean square of the plain logits. float32: sums in another order. bfloat16: activations between
 # the parts are rounded to 8 bits of mantissa.
 TOL = {"float32": 5e-5, "bfloat16": 3e-2}
-# (narrow models average a row's rounding over the fewest elements)
-LOOSER = {"reordered": 1.5, "seed": 2.0}
+# (narrow models average a row's rounding over the fewest elements; "tiled" has scores that are steep in front of their caps:
+# its rows' rounding has a median of 1.6e-2 on every path alike, eager or captured, folded or not, prompt or decoded)
+LOOSER = {"reordered": 1.5, "tiled": 1.25, "seed": 2.0}
 
 
 def row_errors(got, ref):
