@@ -190,10 +190,17 @@ __global__ __launch_bounds__(256, 2) void attention_prefill_kernel(
       s[4 + v] = sb[v];
     }
     if (RULE) {
+      // (the bias as slope * key minus slope * position, so that a score takes one multiply-add for it; the cap's own
+      // cap - 2 cap / (1 + e^2y) starts from it)
+      const float base = (cap2 > 0.f ? cap2 : 0.f) - sl[hh] * (float)(p_mine - key0 - 8 * qd);
+      if (cap2 > 0.f) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) s[e] = cap2 > 0.f ? cap2 * gl3_tanh_of_exponent(s[e] * rule_in) : s[e] * rule_in;
-    }
-    if (BIAS) {
+        for (int e = 0; e < 8; ++e) s[e] = fmaf(-2.0f * cap2, gl3_tanh_part(s[e] * rule_in), fmaf(sl[hh], (float)e, base));
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s[e] = fmaf(s[e], rule_in, fmaf(sl[hh], (float)e, base));
+      }
+    } else if (BIAS) {
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
         const int k1 = key0 + 8 * qd + v;
@@ -435,14 +442,22 @@ __global__ __launch_bounds__(256, OCC) void attention_prefill_wide_kernel(
       }
       if (kk % 4 == 3) __builtin_amdgcn_sched_barrier(0);
     }
-    if (RULE) {
+    if (RULE) {                                 // (as in the kernel above)
+      const float base = (cap2 > 0.f ? cap2 : 0.f) - sl * (float)(p_mine - key0 - 8 * h);
+      if (cap2 > 0.f) {
 #pragma unroll
-      for (int t = 0; t < NT; ++t)
+        for (int t = 0; t < NT; ++t)
 #pragma unroll
-        for (int v = 0; v < 16; ++v)
-          s[t][v] = cap2 > 0.f ? cap2 * gl3_tanh_of_exponent(s[t][v] * rule_in) : s[t][v] * rule_in;
-    }
-    if (BIAS) {
+          for (int v = 0; v < 16; ++v)
+            s[t][v] = fmaf(-2.0f * cap2, gl3_tanh_part(s[t][v] * rule_in), fmaf(sl, (float)(32 * t + 16 * (v >> 3) + (v & 7)), base));
+      } else {
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int v = 0; v < 16; ++v)
+            s[t][v] = fmaf(s[t][v], rule_in, fmaf(sl, (float)(32 * t + 16 * (v >> 3) + (v & 7)), base));
+      }
+    } else if (BIAS) {
 #pragma unroll
       for (int t = 0; t < NT; ++t)
 #pragma unroll

@@ -173,10 +173,9 @@ __device__ __forceinline__ float gl3_query_temperature(int p, const Gl3ScoreRule
   return r.temp_every > 0 ? 1.0f + r.temp_coef * logf((float)((p + 1) / r.temp_every + 1)) : 1.0f;
 }
 // tanh by one exponential and one reciprocal: 1 - 2 / (1 + e^(2y)), given y2 = 2 y log2(e); its error is one of
-// 32-bit rounding of numbers around one (not relative to a small tanh).
-__device__ __forceinline__ float gl3_tanh_of_exponent(float y2) {
-  return fmaf(-2.0f, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(y2)), 1.0f);
-}
+// 32-bit rounding of numbers around one (not relative to a small tanh). gl3_tanh_part: 1 / (1 + e^(2y)) alone.
+__device__ __forceinline__ float gl3_tanh_part(float y2) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(y2)); }
+__device__ __forceinline__ float gl3_tanh_of_exponent(float y2) { return fmaf(-2.0f, gl3_tanh_part(y2), 1.0f); }
 __device__ __forceinline__ float gl3_sigmoid_fast(float z) {
   return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
 }

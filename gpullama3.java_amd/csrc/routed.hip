@@ -209,11 +209,16 @@ struct RowFactors {
   const float* in;
   const float* out;
 };
+// (A kernel brings them into shared memory with its rows, before the products: at the end a row's number, then its
+// factor, would be two more trips to memory.)
+__device__ __forceinline__ void factors_here(const RowFactors& f, int row, float* in, float* out) {
+  *in = f.in && row >= 0 ? f.in[row] : 1.f;
+  *out = f.out && row >= 0 ? f.out[row] : 1.f;
+}
 template <typename TO>
 __device__ __forceinline__ void expert_store(TO* __restrict__ out, long ldo, int row, int n, bool ok, float v, int act,
-                                             int gate_act, float limit, float shift, const RowFactors& f) {
-  if (f.in) v *= ok ? f.in[row] : 0.f;
-  const float after = f.out && ok ? f.out[row] : 1.f;
+                                             int gate_act, float limit, float shift, float before, float after) {
+  v *= before;
   if (gate_act < 0) {
     if (ok) out[(long)row * ldo + n] = from_f32<TO>(gl3_expert_act(v, act) * after);
     return;
@@ -257,10 +262,15 @@ __global__ __launch_bounds__(256) void expert_gemm_generic_kernel(const TA* __re
   __shared__ float sa[EG_TM][EG_TK + 1];
   __shared__ float sw[EG_TN][EG_TK + 1];
   __shared__ int rows[EG_TM];
+  __shared__ float f_in[EG_TM], f_out[EG_TM];
   int e, lo, hi;
   if (!expert_tile(offsets, E, n_rows, EG_TM, blockIdx.x, &e, &lo, &hi)) return;
   const int m = hi - lo < EG_TM ? hi - lo : EG_TM;
-  if (threadIdx.x < EG_TM) rows[threadIdx.x] = threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+  if (threadIdx.x < EG_TM) {
+    const int row = threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+    rows[threadIdx.x] = row;
+    factors_here(rf, row, &f_in[threadIdx.x], &f_out[threadIdx.x]);
+  }
   __syncthreads();
   const int n0 = blockIdx.y * EG_TN;
   const TW* We = W + (long)e * N * K;
@@ -287,7 +297,8 @@ __global__ __launch_bounds__(256) void expert_gemm_generic_kernel(const TA* __re
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int n = n0 + cg + 16 * j;
-    expert_store<TO>(out, ldo, rows[r], n, rows[r] >= 0 && n < N, acc[j], act, gate_act, limit, shift, rf);
+    expert_store<TO>(out, ldo, rows[r], n, rows[r] >= 0 && n < N, acc[j], act, gate_act, limit, shift,
+                     f_in[r], f_out[r]);
   }
 }
 
@@ -306,10 +317,15 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(const bf16_t* __r
                                                                 TO* __restrict__ out, long ldo, int act, int gate_act, float limit,
                                                                    float shift, RowFactors rf) {
   __shared__ int rows[EM_TM];
+  __shared__ float f_in[EM_TM], f_out[EM_TM];
   int e, lo, hi;
   if (!expert_tile(offsets, E, n_rows, EM_TM, blockIdx.x, &e, &lo, &hi)) return;
   const int m = hi - lo < EM_TM ? hi - lo : EM_TM;
-  if (threadIdx.x < EM_TM) rows[threadIdx.x] = threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+  if (threadIdx.x < EM_TM) {
+    const int row = threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+    rows[threadIdx.x] = row;
+    factors_here(rf, row, &f_in[threadIdx.x], &f_out[threadIdx.x]);
+  }
   __syncthreads();
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int li = lane & 15, kb = (lane >> 4) * 4;           // operand row / column of this lane, and its 4 k
@@ -345,8 +361,8 @@ __global__ __launch_bounds__(256) void expert_gemm_mfma_kernel(const bf16_t* __r
   for (int g = 0; g < 4; ++g) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int row = rows[g * 16 + (lane >> 4) * 4 + i];
-      expert_store<TO>(out, ldo, row, nc, row >= 0 && nc < N, acc[g][i], act, gate_act, limit, shift, rf);
+      const int r = g * 16 + (lane >> 4) * 4 + i, row = rows[r];
+      expert_store<TO>(out, ldo, row, nc, row >= 0 && nc < N, acc[g][i], act, gate_act, limit, shift, f_in[r], f_out[r]);
     }
   }
 }
@@ -368,11 +384,16 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
                                                                    float shift, RowFactors rf) {
   constexpr int TM = 16 * G;
   __shared__ int rows[TM];
+  __shared__ float f_in[TM], f_out[TM];
   __shared__ float part[EF_WAVES][TM][EF_TN + 1];
   int e, lo, hi;
   if (!expert_tile(offsets, E, n_rows, TM, blockIdx.x, &e, &lo, &hi)) return;
   const int m = hi - lo < TM ? hi - lo : TM;
-  if (threadIdx.x < TM) rows[threadIdx.x] = (int)threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+  int my_row = -1;
+  if (threadIdx.x < TM) {
+    my_row = (int)threadIdx.x < m ? (sorted ? sorted[lo + threadIdx.x] : lo + threadIdx.x) : -1;
+    rows[threadIdx.x] = my_row;
+  }
   __syncthreads();
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int li = lane & 15, kg = (lane >> 4) * 8;
@@ -387,6 +408,8 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
     const int row = rows[g * 16 + li];                  // (rows beyond the run read the run's first row; their results are dropped)
     ap[g] = A + (long)((row >= 0 ? row : rows[0]) / a_div) * lda + kg;
   }
+  float my_in = 1.f, my_out = 1.f;              // (asked for here, needed at the end)
+  if (threadIdx.x < TM) factors_here(rf, my_row, &my_in, &my_out);
   const bf16x8_few_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
   float4_t acc[G];
 #pragma unroll
@@ -419,6 +442,10 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
     }
   }
   // a lane holds column li of rows 4 (lane / 16) .. + 3 of every group
+  if (threadIdx.x < TM) {
+    f_in[threadIdx.x] = my_in;
+    f_out[threadIdx.x] = my_out;
+  }
 #pragma unroll
   for (int g = 0; g < G; ++g)
 #pragma unroll
@@ -432,7 +459,7 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
 #pragma unroll
     for (int w = 0; w < EF_WAVES; ++w) sum += part[w][r][c];
     const int nc = blockIdx.y * EF_TN + c;
-    expert_store<TO>(out, ldo, rows[r], nc, in && nc < N, sum, act, gate_act, limit, shift, rf);
+    expert_store<TO>(out, ldo, rows[r], nc, in && nc < N, sum, act, gate_act, limit, shift, f_in[r], f_out[r]);
   }
 }
 
@@ -458,11 +485,16 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
   __shared__ __attribute__((aligned(16))) bf16_t As[2][ET_BM][ET_LD];
   __shared__ __attribute__((aligned(16))) bf16_t Ws[2][ET_BN][ET_LD];
   __shared__ int rows[ET_BM];
+  __shared__ float f_in[ET_BM], f_out[ET_BM];
   int e, lo, hi;
   if (!expert_tile(offsets, E, n_rows, ET_BM, blockIdx.x, &e, &lo, &hi)) return;
   const int m = hi - lo < ET_BM ? hi - lo : ET_BM;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  if (tid < ET_BM) rows[tid] = tid < m ? (sorted ? sorted[lo + tid] : lo + tid) : -1;
+  if (tid < ET_BM) {
+    const int row = tid < m ? (sorted ? sorted[lo + tid] : lo + tid) : -1;
+    rows[tid] = row;
+    factors_here(rf, row, &f_in[tid], &f_out[tid]);
+  }
   __syncthreads();
   const int wm = wave / 2, wn = wave % 2;
   const int lr = lane & 31, lh = lane >> 5;
@@ -534,11 +566,11 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
   // a lane holds C[row(v)][col]: row(v) = 8 * (v / 4) + 4 * (lane / 32) + v % 4 inside a 32 x 32 tile, col = lane % 32
 #pragma unroll
   for (int v = 0; v < 16; ++v) {
-    const int row = rows[wm * 32 + (v >> 2) * 8 + lh * 4 + (v & 3)];
+    const int r = wm * 32 + (v >> 2) * 8 + lh * 4 + (v & 3), row = rows[r];
 #pragma unroll
     for (int tn = 0; tn < 2; ++tn) {
       const int n = n0 + wn * 64 + tn * 32 + lr;
-      expert_store<TO>(out, ldo, row, n, row >= 0 && n < N, acc[tn][v], act, gate_act, limit, shift, rf);
+      expert_store<TO>(out, ldo, row, n, row >= 0 && n < N, acc[tn][v], act, gate_act, limit, shift, f_in[r], f_out[r]);
     }
   }
 }
@@ -559,10 +591,13 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
   GL3_REQUIRE(act >= 0 && act <= 3, "gl3_expert_gemm: unknown activation %d", act);
   GL3_REQUIRE((N + 63) / 64 <= 65535, "gl3_expert_gemm: %d columns exceed the grid", N);
   const int e_eff = offsets ? E : 1;
+  // (a product of a few columns, a router's: tiles of 128 columns would leave most of the chip idle; it takes the kernel
+  // for few rows whatever its rows, in tiles of 16 of them)
+  const bool narrow = !offsets && N <= 64;
   // many rows (an expert's run fills tiles of 128): the tiled kernel
   if (use_mfma && a_dtype == GL3_BF16 && w_dtype == GL3_BF16 && K % 8 == 0 && K >= 8 && lda % 8 == 0 &&
       (reinterpret_cast<uintptr_t>(A) % 16 == 0) && (reinterpret_cast<uintptr_t>(W) % 16 == 0) &&
-      n_rows > 64 * e_eff && (out_dtype == GL3_BF16 || out_dtype == GL3_F32)) {
+      n_rows > 64 * e_eff && !narrow && (out_dtype == GL3_BF16 || out_dtype == GL3_F32)) {
     const dim3 grid((n_rows + ET_BM - 1) / ET_BM + (offsets ? E : 0), (N + ET_BN - 1) / ET_BN), block(512);
     if (out_dtype == GL3_BF16)
       expert_gemm_tiled_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
@@ -576,8 +611,8 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
   // few rows (an expert's run is a tile or two): the kernel that reads each weight row in long pieces, K in slices
   if (use_mfma && a_dtype == GL3_BF16 && w_dtype == GL3_BF16 && K % 8 == 0 && lda % 8 == 0 &&
       (reinterpret_cast<uintptr_t>(A) % 16 == 0) && (reinterpret_cast<uintptr_t>(W) % 16 == 0) &&
-      n_rows <= 64 * e_eff && (N + EF_TN - 1) / EF_TN <= 65535 && (out_dtype == GL3_BF16 || out_dtype == GL3_F32)) {
-    const int G = n_rows <= 16 * e_eff ? 1 : n_rows <= 32 * e_eff ? 2 : 4;      // by the runs' mean length
+      (narrow || n_rows <= 64 * e_eff) && (N + EF_TN - 1) / EF_TN <= 65535 && (out_dtype == GL3_BF16 || out_dtype == GL3_F32)) {
+    const int G = n_rows <= 16 * e_eff || narrow ? 1 : n_rows <= 32 * e_eff ? 2 : 4;      // by the runs' mean length
     const dim3 grid((n_rows + 16 * G - 1) / (16 * G) + (offsets ? E : 0), (N + EF_TN - 1) / EF_TN), block(EF_WAVES * 64);
 #define EF_LAUNCH(TO, G)                                                                                                \
   expert_gemm_few_kernel<TO, G><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets, \

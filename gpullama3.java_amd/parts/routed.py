@@ -168,7 +168,11 @@ class RoutedFeedForward:
                 norm = (h.ssq, h.n_partials, d, h.eps)
             else:
                 h = h.materialize()
-        ops.linear(h, self.w_router, logits, ops.EPI_STORE, ctx)
+        if T > 64 and mfma and h.dtype == self.w_router.dtype == torch.bfloat16 and self.w_router.shape[0] <= 64:
+            # many rows and few columns: the experts' kernel that slices K (the tiled product would have a block for 128 rows)
+            K.expert_gemm(h, self.w_router.unsqueeze(0), logits, mfma=True)
+        else:
+            ops.linear(h, self.w_router, logits, ops.EPI_STORE, ctx)
         if norm is not None:
             h = h.xg
         idx = ctx.buffer("router_choice", (T, per), torch.int32)
