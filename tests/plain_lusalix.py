@@ -31,6 +31,17 @@ def silu(z):
     return z * sigmoid(z)
 
 
+def exact(a):
+    return a
+
+
+def to_16_bits(a):
+    """Rounded to bfloat16: what a 16-bit engine does to the activations between its parts. Every function here takes
+    such a rounding as ``r`` (``exact``: none), so that the error that rounding alone makes in a model can be known."""
+    import torch
+    return torch.as_tensor(np.asarray(a, np.float64)).to(torch.bfloat16).double().numpy()
+
+
 def linear(x, w):
     return np.asarray(x, np.float64) @ np.asarray(w, np.float64).T
 
@@ -64,17 +75,17 @@ def blend(v, first, lam):
     return (1.0 - lam) * v + lam * first
 
 
-def attention(h, positions, W, p, m, state, first=None):
+def attention(h, positions, W, p, m, state, first=None, r=exact):
     """``state``: {"k": [n, G, dim], "v": [n, G, vdim]} so far. ``first``: None where the layer's values stay as they
     are, else the values of the same tokens that they are blended with. Returns (output, the values as projected)."""
     T = h.shape[0]
     H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q = linear(h, W[p + "q"]).reshape(T, H, D)
+    q = r(linear(h, W[p + "q"])).reshape(T, H, D)
     if m.get("q_temp") is not None:
         q = q * temperature(positions, m["q_temp"]["coef"], m["q_temp"]["every"])[:, None, None]
-    k = linear(h, W[p + "k"]).reshape(T, G, D)
-    own = linear(h, W[p + "v"]).reshape(T, G, Dv)
-    v = own if first is None else blend(own, first, float(W[p + "vmix"]))
+    k = r(linear(h, W[p + "k"])).reshape(T, G, D)
+    own = r(linear(h, W[p + "v"])).reshape(T, G, Dv)
+    v = own if first is None else r(blend(own, first, float(W[p + "vmix"])))
     state["k"] = k if "k" not in state else np.concatenate([state["k"], k])
     state["v"] = v if "v" not in state else np.concatenate([state["v"], v])
     size = (m.get("mask") or {}).get("size")
@@ -88,13 +99,13 @@ def attention(h, positions, W, p, m, state, first=None):
             s = score(q[t, a], state["k"][lo:i + 1, g], i, j, m, a)
             e = np.exp(s - s.max())
             out[t, a] = (e / e.sum()) @ state["v"][lo:i + 1, g]
-    y = out.reshape(T, H * Dv) * sigmoid(linear(h, W[p + "g"]))
+    y = r(out.reshape(T, H * Dv) * sigmoid(r(linear(h, W[p + "g"]))))
     return linear(y, W[p + "o"]), own
 
 
 # ----------------------------------------------------------------- feed-forward
-def expert(h, W, p):
-    return linear(silu(linear(h, W[p + "gate"])) * linear(h, W[p + "up"]), W[p + "down"])
+def expert(h, W, p, r=exact):
+    return linear(r(silu(linear(h, W[p + "gate"])) * linear(h, W[p + "up"])), W[p + "down"])
 
 
 def route(h, W, p, router):
@@ -104,7 +115,7 @@ def route(h, W, p, router):
     return idx, np.take_along_axis(s, idx, -1), s
 
 
-def mixture(h, W, p, mlp, note=None):
+def mixture(h, W, p, mlp, note=None, r=exact):
     """``note`` (a list) receives, per token, how far the last chosen expert's score lies above the first left out."""
     top = mlp["router"]["top"]
     idx, w, s = route(h, W, p, mlp["router"])
@@ -114,9 +125,9 @@ def mixture(h, W, p, mlp, note=None):
     out = np.zeros_like(h, dtype=np.float64)
     for t in range(h.shape[0]):
         for e, a in zip(idx[t], w[t]):
-            out[t] += expert(a * h[t:t + 1], W, f"{p}e{e}.")[0]
+            out[t] += expert(a * h[t:t + 1], W, f"{p}e{e}.", r)[0]
     if mlp.get("shared") is not None:
-        out += sigmoid(linear(h, W[p + "shared.sg"])) * expert(h, W, p + "shared.")
+        out += sigmoid(linear(h, W[p + "shared.sg"])) * expert(h, W, p + "shared.", r)
     return out
 
 
@@ -125,15 +136,15 @@ class Sequence:
     """One sequence that is fed in pieces. ``rows`` collects, per piece, the residual rows after every layer; ``after``
     (optional) is called with (layer, "mixer" or "ffn", the rows)."""
 
-    def __init__(self, cfg, W, after=None):
-        self.cfg, self.W, self.after = cfg, {k: np.asarray(v, np.float64) for k, v in W.items()}, after
+    def __init__(self, cfg, W, after=None, r=exact):
+        self.cfg, self.W, self.after, self.r = cfg, {k: np.asarray(v, np.float64) for k, v in W.items()}, after, r
         self.n = 0
         self.states = [dict() for _ in cfg["layers"]]
         self.rows = []
         self.gaps = []          # of every router's choices so far (``mixture``)
 
     def feed(self, tokens):
-        cfg, W, eps = self.cfg, self.W, self.cfg["norm"]["eps"]
+        cfg, W, eps, r = self.cfg, self.W, self.cfg["norm"]["eps"], self.r
         positions = np.arange(self.n, self.n + len(tokens))
         self.n += len(tokens)
         x = W["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
@@ -141,20 +152,20 @@ class Sequence:
         for i, lay in enumerate(cfg["layers"]):
             p, m = f"l{i}.", lay["mixer"]
             mixes = bool(m.get("v_mix"))
-            y, own = attention(rms_norm(x, W[p + "norm1"], eps), positions, W, p + "mix.", m, self.states[i],
-                               first if mixes else None)
+            y, own = attention(r(rms_norm(x, W[p + "norm1"], eps)), positions, W, p + "mix.", m, self.states[i],
+                               first if mixes else None, r)
             if mixes and first is None:
                 first = own
             x = x + y
             if self.after:
                 self.after(i, "mixer", x)
             if lay.get("mlp") is not None:
-                x = x + mixture(rms_norm(x, W[p + "norm2"], eps), W, p + "mlp.", lay["mlp"], self.gaps)
+                x = x + mixture(r(rms_norm(x, W[p + "norm2"], eps)), W, p + "mlp.", lay["mlp"], self.gaps, r)
                 if self.after:
                     self.after(i, "ffn", x)
             rows.append(x)
         self.rows.append(np.stack(rows))
-        return linear(rms_norm(x, W["final.norm"], eps), W["head"])
+        return linear(r(rms_norm(x, W["final.norm"], eps)), W["head"])
 
 
 def forward(cfg, W, tokens):
