@@ -468,12 +468,17 @@ __global__ __launch_bounds__(EF_WAVES * 64) void expert_gemm_few_kernel(const bf
 // in shared memory (while a step's products run out of one, the next step's operands go from registers into the other
 // and the step after that travels from memory to registers; one barrier a step; rows padded by 16 bytes against bank
 // conflicts). A's rows are gathered through the run's pairs, and the results go to the pairs' own rows.
+// Blocks with consecutive numbers go to different XCDs, each with a second-level cache of its own. An XCD takes one
+// stretch of an order that walks panels of ET_PANEL row tiles column by column, so that the blocks it holds at a time
+// form a rectangle and share their rows of A and of W (which are mostly one expert's); the stretches are cut from the
+// tiles that exist, not from the most that could, so that all XCDs get as many.
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x16_t __attribute__((ext_vector_type(16)));
 #define ET_BM 128
 #define ET_BN 128
 #define ET_BK 64
 #define ET_LD (ET_BK + 8)
+#define ET_PANEL 8
 template <typename TO>
 __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __restrict__ A, long lda, int a_div,
                                                                  const bf16_t* __restrict__ W, int N, int K,
@@ -486,8 +491,18 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
   __shared__ __attribute__((aligned(16))) bf16_t Ws[2][ET_BN][ET_LD];
   __shared__ int rows[ET_BM];
   __shared__ float f_in[ET_BM], f_out[ET_BM];
+  int n_tiles = 0;
+  if (offsets)
+    for (int i = 0; i < E; ++i) n_tiles += (offsets[i + 1] - offsets[i] + ET_BM - 1) / ET_BM;
+  else
+    n_tiles = (n_rows + ET_BM - 1) / ET_BM;
+  const int col_tiles = (N + ET_BN - 1) / ET_BN, total = n_tiles * col_tiles;
+  const int per_xcd = (total + 7) / 8, at = (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3);
+  if ((int)(blockIdx.x >> 3) >= per_xcd || at >= total) return;
+  const int panel = at / (ET_PANEL * col_tiles), in_panel = at - panel * ET_PANEL * col_tiles;
+  const int height = min(ET_PANEL, n_tiles - panel * ET_PANEL);
   int e, lo, hi;
-  if (!expert_tile(offsets, E, n_rows, ET_BM, blockIdx.x, &e, &lo, &hi)) return;
+  if (!expert_tile(offsets, E, n_rows, ET_BM, panel * ET_PANEL + in_panel % height, &e, &lo, &hi)) return;
   const int m = hi - lo < ET_BM ? hi - lo : ET_BM;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   if (tid < ET_BM) {
@@ -498,7 +513,7 @@ __global__ __launch_bounds__(512) void expert_gemm_tiled_kernel(const bf16_t* __
   __syncthreads();
   const int wm = wave / 2, wn = wave % 2;
   const int lr = lane & 31, lh = lane >> 5;
-  const int n0 = blockIdx.y * ET_BN;
+  const int n0 = in_panel / height * ET_BN;
   const bf16_t* We = W + (long)e * N * K;
   // every load is unconditional: rows beyond the run read the run's first row, columns beyond N the last one,
   // and their results are dropped
@@ -598,7 +613,9 @@ extern "C" int gl3_expert_gemm(const void* A, int a_dtype, long lda, int a_div, 
   if (use_mfma && a_dtype == GL3_BF16 && w_dtype == GL3_BF16 && K % 8 == 0 && K >= 8 && lda % 8 == 0 &&
       (reinterpret_cast<uintptr_t>(A) % 16 == 0) && (reinterpret_cast<uintptr_t>(W) % 16 == 0) &&
       n_rows > 64 * e_eff && !narrow && (out_dtype == GL3_BF16 || out_dtype == GL3_F32)) {
-    const dim3 grid((n_rows + ET_BM - 1) / ET_BM + (offsets ? E : 0), (N + ET_BN - 1) / ET_BN), block(512);
+    const long most = ((long)(n_rows + ET_BM - 1) / ET_BM + (offsets ? E : 0)) * ((N + ET_BN - 1) / ET_BN);
+    GL3_REQUIRE(most < (1L << 30), "gl3_expert_gemm: %ld tiles exceed the grid", most);
+    const dim3 grid((unsigned)((most + 7) / 8 * 8)), block(512);
     if (out_dtype == GL3_BF16)
       expert_gemm_tiled_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)A, lda, a_div, (const bf16_t*)W, N, K, offsets,
                                                                    sorted, E, n_rows, (bf16_t*)out, ldo, act, gate_act, limit, shift, rf);
