@@ -9,9 +9,11 @@ from .nodupel import NodupelConfiguration
 from .nolatar import NolatarConfiguration
 from .dotanex import DotanexConfiguration
 from .lusalix import LusalixConfiguration
+from .banazen import BanazenConfiguration
 
 __all__ = ["ConfigError", "config_from_dict", "load_config", "register_architecture",
            "registered_architectures", "AttentionSpec", "BlockSpec", "GatedFeedForwardSpec",
            "Llama3RopeScaling", "ModelSpec", "NormSpec", "RotarySpec", "Run", "LlamaConfiguration", "DistanceBias", "GatedDeltaSpec", "Inject",
            "MelizenConfiguration", "NodupelConfiguration", "LinearRopeScaling", "MinGRUSpec", "PairEmbedding", "Remix",
-           "SideBySideSpec", "TimeMixSpec", "NolatarConfiguration", "DotanexConfiguration", "LusalixConfiguration"]
+           "SideBySideSpec", "TimeMixSpec", "NolatarConfiguration", "DotanexConfiguration", "LusalixConfiguration",
+           "BanazenConfiguration"]

@@ -131,7 +131,8 @@ class AttentionSpec:
     out_mult: float = 1.0             # a constant that the mixer's output is multiplied by
     qk_norm_eps: Optional[float] = None   # queries and keys are divided by their root mean square per head (this eps
                                       # inside the root) and multiplied by the stored [head_dim] weights ``q_norm`` /
-                                      # ``k_norm`` (shared by the heads) before the rotation; None: no such norm
+                                      # ``k_norm`` (shared by the heads) before the rotation; None: no such norm. Without
+                                      # these names there is no weight (before or behind the rotation is then the same)
     chunk: Optional[int] = None       # n: query i sees key j <= i only if i // n == j // n (chunks count from position 0)
     differential: Optional[Differential] = None
     values_are_keys: bool = False     # no value projection: a position's values are its keys as projected (before the
@@ -139,6 +140,9 @@ class AttentionSpec:
     score_softcap: Optional[float] = None     # the scaled score becomes cap * tanh(score / cap), before any distance bias is taken off
     query_temperature: Optional[QueryTemperature] = None
     value_mix: Optional[ValueMix] = None
+    conv_taps: int = 0                # n: each channel of q, k and v passes a causal convolution over time right behind its
+                                      # projection, ``y_t = sum_j w[:, j] u_(t - n + 1 + j)`` with zeros before the sequence's
+                                      # start (names ``q_conv``, ``k_conv``, ``v_conv``: [channels, n]); 0: none
     # (a name ``gate`` among ``names``: a stored [n_heads * v_head_dim, hidden] matrix; the heads' outputs together are
     # multiplied element by element with sigmoid of its product with the mixer's input, before the output projection)
     # (a name ``sink`` among ``names``: a stored [n_heads] vector, a learned sink per query head in place of ``sink``)
@@ -194,10 +198,11 @@ class SideBySideSpec:
 class LatentAttentionSpec:
     """Causal attention whose keys and values are expanded from one latent per position (``parts/latent_attention.py``).
     Queries: ``c_q = RMSnorm(W_dq h)`` (``q_rank`` elements), ``q = W_uq c_q``, per head [``head_dim`` unrotated |
-    ``rot_dim`` rotated]. ``W_dkv h`` gives the latent c (``kv_rank``, RMS-normed) and ``rot_dim`` more elements, one
+    ``rot_dim`` rotated]; with ``q_rank`` 0 ``q = W_q h`` (name ``q``). ``W_dkv h`` gives the latent c (``kv_rank``, RMS-normed) and ``rot_dim`` more elements, one
     rotated key part for all heads. Per head the unrotated key is ``W_uk c`` and the value ``W_uv c``
     (``v_head_dim``); score = (q . k over both parts) * ``scale``; an ordinary softmax; the heads' outputs times
-    sigmoid of a gate projection of the mixer's input; output projection. Only c and the rotated part are cached."""
+    sigmoid of a gate projection of the mixer's input (no name ``g``: no gate); output projection. Only c and the rotated
+    part are cached. Without the name ``dkv`` the mixer has no latents of its own and only ever reads another entry's."""
     kind: str = "latent_attention"
     hidden: int = 0
     n_heads: int = 0
@@ -209,8 +214,11 @@ class LatentAttentionSpec:
     scale: float = 1.0
     position: Optional[RotarySpec] = None      # over the rot_dim part
     norm_eps: float = 1e-5
-    names: dict = field(default_factory=dict)  # "dq", "dq_norm", "uq", "dkv", "dkv_norm", "uk", "uv", "g", "o"
+    names: dict = field(default_factory=dict)  # "dq", "dq_norm", "uq" (or "q"), "dkv", "dkv_norm", "uk", "uv", "g", "o"
     out_mult: float = 1.0
+    window: Optional[int] = None      # None: every earlier key; n: the last n keys
+    kept_window: Optional[int] = None # with ``window``: how far back the cache holds this layer's latents where other layers
+                                      # read them through wider windows (0: to the sequence's start); None: ``window``
 
 
 @dataclass(frozen=True)
@@ -261,7 +269,10 @@ class StateSpaceSpec:
 class GatedDeltaSpec:
     """The gated delta rule: per value head a matrix [key_dim, value_dim] in 32-bit that every token decays,
     corrects towards its value along its key, and reads with its query (``parts/delta.py``). ``n_heads`` value
-    heads share ``n_kv_heads`` query/key heads; q, k and v pass a causal convolution of ``conv_taps`` taps."""
+    heads share ``n_kv_heads`` query/key heads; q, k and v pass a causal convolution of ``conv_taps`` taps. With a
+    ``decay_rank`` every row of a head's matrix decays by itself, ``exp(-exp(A_log_h) softplus(W_a2 (W_a1 h) +
+    dt_bias))`` with names ``a1`` [rank, hidden], ``a2`` and ``dt_bias`` over heads x key_dim in place of ``a``; with a
+    ``gate_rank`` the read-out's gate is ``W_g2 (W_g1 h)`` (names ``g1``, ``g2`` in place of ``g``)."""
     kind: str = "gated_delta"
     hidden: int = 0
     n_heads: int = 0
@@ -273,6 +284,9 @@ class GatedDeltaSpec:
     norm_eps: float = 1e-5            # the read-out's norm
     names: dict = field(default_factory=dict)
     out_scale_name: Optional[str] = None
+    decay_rank: int = 0               # 0: one decay per head
+    gate_rank: int = 0                # 0: the gate is one projection
+    gate_activation: str = "silu"     # "silu" or "sigmoid" of the gate
 
 
 @dataclass(frozen=True)
@@ -322,6 +336,10 @@ class RoutedFeedForwardSpec:
     # sum plus ``sum_eps``. "chosen_softmax": the softmax over the chosen logits alone.
     weights: str = "chosen_softmax"
     sum_eps: float = 0.0
+    # (with "scores") the experts form ``groups[0]`` equal groups of neighbours, of which the ``groups[1]`` whose largest
+    # choice score is largest stay open; only their experts can be chosen. None: all are open
+    groups: Optional[tuple] = None
+    weight_scale: float = 1.0         # a constant on the chosen experts' weights (not on the shared expert's)
     n_identity: int = 0               # the router's last outputs stand for experts whose output is their input (no tensors);
                                       # the router has n_experts + n_identity rows
     # A third rule (``weights = "sigmoid"``): the ``top`` largest router outputs are chosen, each weighted with its own
@@ -330,6 +348,22 @@ class RoutedFeedForwardSpec:
     # (a name ``shared_weight``: a stored [1, hidden] row; the shared expert's output is multiplied by sigmoid of its
     # product with the token's input)
     # (names: ``expert_gate`` beside ``expert_up`` / ``expert_down`` for gated experts, ``shared_gate``; ``correction``)
+
+
+@dataclass(frozen=True)
+class TokenSideSpec:
+    """What a token's own row of a side table adds behind a layer's sublayers (``parts/token_side.py``): with e the
+    columns ``index * dim ..`` of row ``token`` of the stored table ``embed`` [``rows``, ``columns``],
+    ``g = act(W_gate x) * e; y = W_proj g; x <- x + y / rms(y) * norm`` (eps inside the root). x is the residual row itself."""
+    kind: str = "token_side"
+    hidden: int = 0
+    dim: int = 0
+    rows: int = 0
+    columns: int = 0
+    index: int = 0
+    activation: str = "gelu_tanh"
+    norm_eps: float = 1e-5
+    names: dict = field(default_factory=dict)     # "embed", "gate", "proj", "norm"
 
 
 @dataclass(frozen=True)
@@ -346,6 +380,7 @@ class BlockSpec:
     mixer: object = None
     ffn_norm: object = None
     ffn: object = None
+    side: object = None               # a part that adds to the residual rows behind the sublayers ("prenorm", "parallel")
     streams: int = 1
     stream_names: dict = field(default_factory=dict)
 

@@ -16,7 +16,10 @@
 //
 // Two entry points: delta_prep (convolution, silu, unit length, decay and strength; then the convolution's new
 // state) and delta_recurrence (the rule itself, then each head's read-out divided by its root mean square, times a
-// weight shared by the heads, times silu of a gate).
+// weight shared by the heads, times silu or sigmoid of a gate).
+//
+// A decay per key channel instead of one per head: S <- diag(g) S, g of D numbers a head and token. delta_inner makes
+// them, and the read-out's gate, from two-step projections: g = exp(-exp(A_log[h]) softplus(W_a2 (W_a1 h) + dt_bias)).
 #include "common.h"
 
 __device__ __forceinline__ float dr_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
@@ -42,8 +45,10 @@ __global__ __launch_bounds__(64) void delta_prep_kernel(
   const float* row = proj + (long)t * s.ldp;
   if (u == 2 * s.G + s.H) {
     for (int h = lane; h < s.H; h += 64) {
-      const float sp = dr_softplus(row[s.off_a + h] + dt_bias[h]);
-      gates[(long)t * 2 * s.H + h] = expf(-expf(A_log[h]) * sp);
+      if (A_log) {      // (null: the decays are per key channel and come from elsewhere)
+        const float sp = dr_softplus(row[s.off_a + h] + dt_bias[h]);
+        gates[(long)t * 2 * s.H + h] = expf(-expf(A_log[h]) * sp);
+      }
       gates[(long)t * 2 * s.H + s.H + h] = dr_sigmoid(row[s.off_b + h]);
     }
     return;
@@ -109,7 +114,8 @@ __global__ __launch_bounds__(256) void delta_conv_state_kernel(const float* __re
 // After the last token the block divides each of its tokens' read-outs (which it wrote to `o` itself) by their
 // root mean square over the head and applies the weight and the gate: y = o / rms * w * silu(gate).
 #define DR_CHUNK 16   // the most tokens a chunk; the launcher takes fewer where keys and values are long
-#define DR_NLD 8       // loads a thread has on their way for the next chunk
+#define DR_NLD 8       // loads a thread has on their way for the next chunk (with decays per channel DR_NLD_CH)
+#define DR_NLD_CH 10
 
 __device__ __forceinline__ float dr_sum4(float p) {   // the sum over lanes l, l ^ 16, l ^ 32, l ^ 48
   auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(p), __float_as_uint(p), false, false);
@@ -127,12 +133,16 @@ __device__ __forceinline__ float dr_sum_rows(float p) {
   return dr_sum4(p);
 }
 
-template <int RPL, typename TO, int MAXT, int RG>
+__device__ __forceinline__ float dr_gate(float z, int sigmoid) { return sigmoid ? dr_sigmoid(z) : z * dr_sigmoid(z); }
+
+// CH: decay [T][H D] holds a factor per key channel, a third operand of D numbers beside k and q.
+template <int RPL, typename TO, int MAXT, int RG, bool CH>
 __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
-    const float* __restrict__ act, const float* __restrict__ gates, float* __restrict__ state,
+    const float* __restrict__ act, const float* __restrict__ gates, const float* __restrict__ decay, float* __restrict__ state,
     const int* __restrict__ cu_seqlens, const int* __restrict__ slot_ids, float* __restrict__ o,
     const float* __restrict__ proj, int ldp, int off_gate, const float* __restrict__ norm_w, TO* __restrict__ y,
-    float eps, DeltaShape s, int chunk, int norm_here, int own_waves) {
+    float eps, DeltaShape s, int chunk, int norm_here, int own_waves, int gate_sigmoid) {
+  constexpr int NLD = CH ? DR_NLD_CH : DR_NLD;
   extern __shared__ __attribute__((aligned(16))) float dr_lds[];   // two buffers of chunk * per_token floats
   typedef float f4 __attribute__((ext_vector_type(4)));
   const int h = blockIdx.x, b = blockIdx.y;
@@ -156,44 +166,46 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
     const int i = r + RG * ii;
     S[ii] = (owner && i < D) ? tile[(long)i * 16] : 0.f;
   }
-  // A token's operands in a chunk's buffer: q | k | v [Dv] | decay, strength, where q and k lie as the lanes read
+  // A token's operands in a chunk's buffer: q | k (| decays) | v [Dv] | decay, strength, where q and k lie as the lanes read
   // them: row r + RG ii at [r][ii], RPL places a lane (rows beyond D stay zero), so a lane's share is 16-byte reads.
-  const int per_src = 2 * D + Dv + 2;                           // what a token brings
+  constexpr int NV = CH ? 3 : 2;                                // vectors over the key channels
+  const int per_src = NV * D + Dv + (CH ? 1 : 2);               // what a token brings
   constexpr int VEC = RG * RPL;                                 // places of q, and of k
-  const int per_token = 2 * VEC + ((Dv + 2 + 3) & ~3);          // what it takes in the buffer
+  const int per_token = NV * VEC + ((Dv + 2 + 3) & ~3);         // what it takes in the buffer
   const int n_src = chunk * per_src;
   const long q_at = (long)kvh * D, k_at = (long)s.G * D + (long)kvh * D, v_at = 2L * s.G * D + (long)h * Dv;
   const int threads = blockDim.x;
   for (int e = tid; e < 2 * chunk * per_token; e += threads) dr_lds[e] = 0.f;
   __syncthreads();
-  float held[DR_NLD];
+  float held[NLD];
   auto ask = [&](int t0) {
 #pragma unroll
-    for (int n = 0; n < DR_NLD; ++n) {
+    for (int n = 0; n < NLD; ++n) {
       const int e = tid + n * threads;
       const int tt = e / per_src, f = e - tt * per_src, t = t0 + tt;
       const float* p = act;
       if (e < n_src && t < last) {
         if (f < D) p = act + (long)t * C + q_at + f;
         else if (f < 2 * D) p = act + (long)t * C + k_at + (f - D);
-        else if (f < 2 * D + Dv) p = act + (long)t * C + v_at + (f - 2 * D);
-        else p = gates + (long)t * 2 * H + (long)(f - 2 * D - Dv) * H + h;
+        else if (CH && f < 3 * D) p = decay + (long)t * H * D + (long)h * D + (f - 2 * D);
+        else if (f < NV * D + Dv) p = act + (long)t * C + v_at + (f - NV * D);
+        else p = gates + (long)t * 2 * H + (long)(CH ? 1 : f - 2 * D - Dv) * H + h;
       }
       held[n] = *p;
     }
   };
   auto put = [&](int buf) {
 #pragma unroll
-    for (int n = 0; n < DR_NLD; ++n) {
+    for (int n = 0; n < NLD; ++n) {
       const int e = tid + n * threads;
       if (e < n_src) {
         const int tt = e / per_src, f = e - tt * per_src;
         int at;
-        if (f < 2 * D) {
-          const int which = f >= D, i = f - which * D;
+        if (f < NV * D) {
+          const int which = CH && f >= 2 * D ? 2 : f >= D, i = f - which * D;
           at = which * VEC + (i % RG) * RPL + i / RG;
         } else {
-          at = 2 * VEC + (f - 2 * D);
+          at = NV * VEC + (f - NV * D);
         }
         dr_lds[(buf * chunk + tt) * per_token + at] = held[n];
       }
@@ -209,7 +221,7 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
     const int n_here = min(chunk, last - t0);
     // two tokens' operands in registers in turn: the next token's reads from shared memory are on their way while
     // the current token's chain of multiply-adds runs
-    struct Operands { float k[RPL], q[RPL], v, g, beta; };
+    struct Operands { float k[RPL], q[RPL], gs[CH ? RPL : 1], v, beta; };
     auto fetch = [&](Operands& x, int tt) {
       const float* op = dr_lds + (buf * chunk + tt) * per_token;
 #pragma unroll
@@ -217,16 +229,21 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
         const f4 q4 = *(const f4*)(op + r * RPL + ii), k4 = *(const f4*)(op + VEC + r * RPL + ii);
 #pragma unroll
         for (int e = 0; e < 4; ++e) { x.q[ii + e] = q4[e]; x.k[ii + e] = k4[e]; }
+        if constexpr (CH) {
+          const f4 g4 = *(const f4*)(op + 2 * VEC + r * RPL + ii);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) x.gs[ii + e] = g4[e];
+        }
       }
-      x.g = op[2 * VEC + Dv];
-      x.beta = op[2 * VEC + Dv + 1];
-      x.v = valid ? op[2 * VEC + j] : 0.f;
+      if constexpr (!CH) x.gs[0] = op[NV * VEC + Dv];
+      x.beta = op[NV * VEC + Dv + (CH ? 0 : 1)];
+      x.v = valid ? op[NV * VEC + j] : 0.f;
     };
     auto work = [&](const Operands& x, int tt) {
       float p4[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ii = 0; ii < RPL; ++ii) {
-        S[ii] *= x.g;
+        S[ii] *= x.gs[CH ? ii : 0];
         p4[ii & 3] = fmaf(S[ii], x.k[ii], p4[ii & 3]);
       }
       const float part = dr_sum_rows<RG>((p4[0] + p4[1]) + (p4[2] + p4[3]));
@@ -240,7 +257,7 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
       const float read = dr_sum_rows<RG>((o4[0] + o4[1]) + (o4[2] + o4[3]));
       if (r == 0 && valid) o[(long)(t0 + tt) * H * Dv + (long)h * Dv + j] = read;
     };
-    if constexpr (RPL <= 24 && MAXT <= 512) {
+    if constexpr (RPL <= (CH ? 16 : 24) && MAXT <= 512) {
       // (pairs of tokens without a branch between them, so that the end of one token's work, which nothing waits
       // for, can be scheduled into the start of the next one's)
       Operands xa, xb;
@@ -288,16 +305,17 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
     TO* dst = y + ((long)t * H + h) * Dv;
     for (int e = lane; e < Dv; e += 64) {
       const float z = grow[e];
-      dst[e] = from_f32<TO>(orow[e] * f * norm_w[e] * (z * dr_sigmoid(z)));
+      dst[e] = from_f32<TO>(orow[e] * f * norm_w[e] * dr_gate(z, gate_sigmoid));
     }
   }
 }
 
-// grid (T, H), one wave: y[t, h, :] = o / sqrt(mean(o^2) + eps) * w * silu(gate[t, h, :])
+// grid (T, H), one wave: y[t, h, :] = o / sqrt(mean(o^2) + eps) * w * silu(gate[t, h, :]) (or sigmoid of it)
 template <typename TO>
 __global__ __launch_bounds__(64) void delta_gated_norm_kernel(const float* __restrict__ o, const float* __restrict__ proj,
                                                               int ldp, int off_gate, const float* __restrict__ w,
-                                                              TO* __restrict__ y, int H, int Dv, float eps) {
+                                                              TO* __restrict__ y, int H, int Dv, float eps,
+                                                              int gate_sigmoid) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const float* orow = o + ((long)t * H + h) * Dv;
   const float* grow = proj + (long)t * ldp + off_gate + (long)h * Dv;
@@ -308,7 +326,7 @@ __global__ __launch_bounds__(64) void delta_gated_norm_kernel(const float* __res
   TO* dst = y + ((long)t * H + h) * Dv;
   for (int e = lane; e < Dv; e += 64) {
     const float z = grow[e];
-    dst[e] = from_f32<TO>(orow[e] * f * w[e] * (z * dr_sigmoid(z)));
+    dst[e] = from_f32<TO>(orow[e] * f * w[e] * dr_gate(z, gate_sigmoid));
   }
 }
 
@@ -333,13 +351,14 @@ extern "C" long gl3_delta_state_floats(int H, int G, int D, int Dv, int taps) {
 // proj [T][ldp] float: the projection of the step's tokens. conv_w [C][taps], A_log [H], dt_bias [H] float.
 // state [slots][state_stride] float. act [T][C] and gates [T][2 H] float are written; then the held inputs move on
 // (one_each: the caller vouches that every sequence brings exactly one token, and they move on in the same launch).
+// A_log and dt_bias null: no decays per head (gates then holds the strengths in its second half only).
 extern "C" int gl3_delta_prep(const float* proj, const float* conv_w, const float* A_log, const float* dt_bias,
                               float* state, const int* cu_seqlens, const int* seq_of_token, const int* slot_ids,
                               float* act, float* gates, int T, int B, int H, int G, int D, int Dv, int taps, int ldp,
                               int off_q, int off_k, int off_v, int off_b, int off_a, long state_stride, float unit_eps,
                               float q_scale, int one_each, hipStream_t stream) {
   if (T == 0 || B == 0) return 0;
-  GL3_REQUIRE(proj && conv_w && A_log && dt_bias && state && cu_seqlens && seq_of_token && slot_ids && act && gates &&
+  GL3_REQUIRE(proj && conv_w && (A_log == nullptr) == (dt_bias == nullptr) && state && cu_seqlens && seq_of_token && slot_ids && act && gates &&
                   T > 0 && B > 0, "gl3_delta_prep: bad arguments");
   DeltaShape s;
   if (delta_shape(s, H, G, D, Dv, taps, ldp, off_q, off_k, off_v, off_b, off_a, state_stride)) return -1;
@@ -358,11 +377,12 @@ extern "C" int gl3_delta_prep(const float* proj, const float* conv_w, const floa
 
 // act [T][C], gates [T][2 H] as gl3_delta_prep left them. o [T][H Dv] float receives the raw read-outs (scratch);
 // y [T][H Dv] (float or bfloat16) the read-outs divided by their root mean square over each head, times norm_w [Dv]
-// (float), times silu of the gate, whose H Dv columns start at off_gate of proj [T][ldp] (float).
-extern "C" int gl3_delta_recurrence(const float* act, const float* gates, float* state, const int* cu_seqlens,
+// (float), times silu of the gate (gate_sigmoid: sigmoid), whose H Dv columns start at off_gate of proj [T][ldp] (float).
+// decay [T][H D] (may be null): a factor per key channel, in place of the heads' decays in gates.
+extern "C" int gl3_delta_recurrence(const float* act, const float* gates, const float* decay, float* state, const int* cu_seqlens,
                                     const int* slot_ids, float* o, const float* proj, int ldp, int off_gate,
                                     const float* norm_w, void* y, int y_dtype, float eps, int T, int B, int H, int G, int D,
-                                    int Dv, int taps, long state_stride, hipStream_t stream) {
+                                    int Dv, int taps, long state_stride, int gate_sigmoid, hipStream_t stream) {
   if (B == 0 || T == 0) return 0;
   GL3_REQUIRE(act && gates && state && cu_seqlens && slot_ids && o && proj && norm_w && y && B > 0,
               "gl3_delta_recurrence: bad arguments");
@@ -387,21 +407,29 @@ extern "C" int gl3_delta_recurrence(const float* act, const float* gates, float*
   const int all_col_waves = (Dv + cols - 1) / cols;
   const int col_waves = all_col_waves;
   const int split = 1;
+  const int nv = decay ? 3 : 2, nld = decay ? DR_NLD_CH : DR_NLD, per_src = nv * D + Dv + (decay ? 1 : 2);
   int chunk = DR_CHUNK, waves = col_waves;
+  const int rows = (D + rg - 1) / rg;
+  const int rpl = rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : rows <= 24 ? 24 : rows <= 32 ? 32 : rows <= 48 ? 48 : 64;
+  const size_t lds_token = 2 * (size_t)(nv * rg * rpl + ((Dv + 2 + 3) & ~3)) * sizeof(float);
   for (;; chunk /= 2) {
     waves = col_waves;
-    while (waves * 64 * DR_NLD < chunk * (2 * D + Dv + 2)) ++waves;
-    if (waves <= (col_waves > 4 ? col_waves : 4) || chunk == 1) break;
+    while (waves * 64 * nld < chunk * per_src) ++waves;
+    if ((waves <= (col_waves > 4 ? col_waves : 4) && chunk * lds_token <= 64 * 1024) || chunk == 1) break;
   }
   GL3_REQUIRE(waves <= 16, "gl3_delta_recurrence: keys of %d with values of %d need more than a block's threads", D, Dv);
   dim3 grid(H, B, split), block(waves * 64);
-  const int rows = (D + rg - 1) / rg;
-  const int rpl = rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : rows <= 24 ? 24 : rows <= 32 ? 32 : rows <= 48 ? 48 : 64;
-  const size_t lds = 2 * (size_t)chunk * (2 * rg * rpl + ((Dv + 2 + 3) & ~3)) * sizeof(float);
+  const size_t lds = chunk * lds_token;
   GL3_REQUIRE(lds <= 64 * 1024, "gl3_delta_recurrence: a chunk's operands of %zu bytes exceed shared memory", lds);
-#define GO4(R, TO, MAXT, RGV)                                                                                                  \
-  delta_recurrence_kernel<R, TO, MAXT, RGV><<<grid, block, lds, stream>>>(act, gates, state, cu_seqlens, slot_ids, o, proj, ldp, \
-                                                                          off_gate, norm_w, (TO*)y, eps, s, chunk, norm_here, col_waves)
+#define GO5(R, TO, MAXT, RGV, CH)                                                                                          \
+  delta_recurrence_kernel<R, TO, MAXT, RGV, CH><<<grid, block, lds, stream>>>(                                             \
+      act, gates, decay, state, cu_seqlens, slot_ids, o, proj, ldp, off_gate, norm_w, (TO*)y, eps, s, chunk, norm_here,    \
+      col_waves, gate_sigmoid)
+#define GO4(R, TO, MAXT, RGV)                                                  \
+  do {                                                                         \
+    if (decay) GO5(R, TO, MAXT, RGV, true);                                    \
+    else GO5(R, TO, MAXT, RGV, false);                                         \
+  } while (0)
 #define GO3(R, TO, MAXT)                                                       \
   do {                                                                         \
     if constexpr (R <= 32) {                                                   \
@@ -433,13 +461,117 @@ extern "C" int gl3_delta_recurrence(const float* act, const float* gates, float*
 #undef GO2
 #undef GO3
 #undef GO4
+#undef GO5
   GL3_LAUNCH_CHECK();
   if (!norm_here) {
     GL3_REQUIRE(T <= 2147483647 / 64, "gl3_delta_recurrence: %d tokens exceed the grid", T);
     if (y_dtype == GL3_F32)
-      delta_gated_norm_kernel<float><<<dim3(T, H), dim3(64), 0, stream>>>(o, proj, ldp, off_gate, norm_w, (float*)y, H, Dv, eps);
+      delta_gated_norm_kernel<float><<<dim3(T, H), dim3(64), 0, stream>>>(o, proj, ldp, off_gate, norm_w, (float*)y, H, Dv, eps,
+                                                                                 gate_sigmoid);
     else
-      delta_gated_norm_kernel<bf16_t><<<dim3(T, H), dim3(64), 0, stream>>>(o, proj, ldp, off_gate, norm_w, (bf16_t*)y, H, Dv, eps);
+      delta_gated_norm_kernel<bf16_t><<<dim3(T, H), dim3(64), 0, stream>>>(o, proj, ldp, off_gate, norm_w, (bf16_t*)y, H, Dv, eps,
+                                                                                  gate_sigmoid);
+  }
+  GL3_LAUNCH_CHECK();
+  return 0;
+}
+
+// ----------------------------------------------------------------- decays per key channel and the gate, two-step projections
+// proj [T][ldp] float: the first steps' sums, ra columns from col_a (decays) and rg from col_g (gate). w2 [Na + Ng][Rp]: the
+// second steps' rows, the decays' first (padded with zero rows to Na, a multiple of 64), then the gate's (padded to Ng, a
+// multiple of 64), zeros behind each row's ra or rg numbers up to Rp, a multiple of 32.
+//   decay [T][HD] = exp(-exp(A_log[n / D]) softplus(sum + dt_bias[n])),  gate [T][HV] = sum
+// A block takes 64 columns of w2 for 16 MT tokens; the first steps' sums are rounded to the weights' type, as any
+// product's input is.
+struct DeltaInner {
+  int ldp, col_a, ra, col_g, rg, Rp, Na, HD, HV, D, T;
+};
+__device__ __forceinline__ void inner_store(float v, int t, int n, const DeltaInner& s, const float* __restrict__ A_log,
+                                            const float* __restrict__ dt_bias, float* __restrict__ decay, float* __restrict__ gate) {
+  if (t >= s.T) return;
+  if (n < s.Na) {
+    if (n < s.HD) decay[(long)t * s.HD + n] = expf(-expf(A_log[n / s.D]) * dr_softplus(v + dt_bias[n]));
+  } else if (n - s.Na < s.HV) {
+    gate[(long)t * s.HV + n - s.Na] = v;
+  }
+}
+
+typedef __bf16 di_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float di_f32x4 __attribute__((ext_vector_type(4)));
+template <int MT>
+__global__ __launch_bounds__(256) void delta_inner_mfma_kernel(const float* __restrict__ proj, const bf16_t* __restrict__ w2,
+                                                               const float* __restrict__ A_log, const float* __restrict__ dt_bias,
+                                                               float* __restrict__ decay, float* __restrict__ gate, DeltaInner s) {
+  extern __shared__ __attribute__((aligned(16))) char di_smem[];
+  bf16_t* As = reinterpret_cast<bf16_t*>(di_smem);            // [16 MT][Rp + 8]
+  const int lda = s.Rp + 8;
+  const int n0 = blockIdx.x * 64, t0 = blockIdx.y * 16 * MT;
+  const int col = n0 < s.Na ? s.col_a : s.col_g, r = n0 < s.Na ? s.ra : s.rg;
+  for (int i = threadIdx.x; i < 16 * MT * s.Rp; i += 256) {
+    const int row = i / s.Rp, k = i % s.Rp;
+    As[row * lda + k] = static_cast<bf16_t>(k < r && t0 + row < s.T ? proj[(long)(t0 + row) * s.ldp + col + k] : 0.f);
+  }
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, li = lane & 15, lq = lane >> 4;
+  const int n = n0 + wave * 16 + li;
+  const bf16_t* wp = w2 + (long)n * s.Rp + 8 * lq;
+  di_f32x4 acc[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) acc[m] = di_f32x4{0.f, 0.f, 0.f, 0.f};
+  __syncthreads();
+  for (int k = 0; k < s.Rp; k += 32) {
+    const di_bf16x8 b = *reinterpret_cast<const di_bf16x8*>(wp + k);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      const di_bf16x8 a = *reinterpret_cast<const di_bf16x8*>(As + (16 * m + li) * lda + k + 8 * lq);
+      acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[m], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) inner_store(acc[m][i], t0 + 16 * m + 4 * lq + i, n, s, A_log, dt_bias, decay, gate);
+}
+
+__global__ __launch_bounds__(256) void delta_inner_f32_kernel(const float* __restrict__ proj, const float* __restrict__ w2,
+                                                              const float* __restrict__ A_log, const float* __restrict__ dt_bias,
+                                                              float* __restrict__ decay, float* __restrict__ gate, DeltaInner s) {
+  const int n = blockIdx.x * 64 + (threadIdx.x & 63), t = blockIdx.y * 4 + (threadIdx.x >> 6);
+  if (t >= s.T) return;
+  const int col = n < s.Na ? s.col_a : s.col_g, r = n < s.Na ? s.ra : s.rg;
+  const float* a = proj + (long)t * s.ldp + col;
+  const float* w = w2 + (long)n * s.Rp;
+  float v = 0.f;
+  for (int k = 0; k < r; ++k) v = fmaf(a[k], w[k], v);
+  inner_store(v, t, n, s, A_log, dt_bias, decay, gate);
+}
+
+extern "C" int gl3_delta_inner(const float* proj, int ldp, int col_a, int ra, int col_g, int rg, const void* w2, int w_dtype,
+                               int Rp, int Na, int Ng, const float* A_log, const float* dt_bias, float* decay, float* gate,
+                               int T, int H, int D, int Dv, hipStream_t stream) {
+  if (T == 0) return 0;
+  GL3_REQUIRE(proj && w2 && A_log && dt_bias && decay && gate && T > 0 && H > 0 && D > 0 && Dv > 0, "gl3_delta_inner: bad arguments");
+  GL3_REQUIRE(ra > 0 && rg > 0 && Rp % 32 == 0 && ra <= Rp && rg <= Rp && Rp <= 1024, "gl3_delta_inner: inner sizes %d and %d in rows of %d",
+              ra, rg, Rp);
+  GL3_REQUIRE(col_a >= 0 && col_g >= 0 && col_a + ra <= ldp && col_g + rg <= ldp, "gl3_delta_inner: columns beyond the rows of %d", ldp);
+  GL3_REQUIRE(Na % 64 == 0 && Ng % 64 == 0 && Na >= H * D && Ng >= H * Dv && (uintptr_t)w2 % 16 == 0,
+              "gl3_delta_inner: %d and %d rows for %d heads of %d and %d", Na, Ng, H, D, Dv);
+  const DeltaInner s{ldp, col_a, ra, col_g, rg, Rp, Na, H * D, H * Dv, D, T};
+  const unsigned nb = (unsigned)((Na + Ng) / 64);
+  if (w_dtype == GL3_F32) {
+    GL3_REQUIRE((T + 3) / 4 <= 65535, "gl3_delta_inner: %d tokens exceed the grid", T);
+    delta_inner_f32_kernel<<<dim3(nb, (T + 3) / 4), dim3(256), 0, stream>>>(proj, (const float*)w2, A_log, dt_bias, decay, gate, s);
+  } else if (w_dtype == GL3_BF16) {
+    const int mt = T <= 16 ? 1 : 4;
+    const size_t lds = (size_t)16 * mt * (Rp + 8) * sizeof(bf16_t);
+    GL3_REQUIRE((T + 16 * mt - 1) / (16 * mt) <= 65535 && (lds <= 64 * 1024 || mt > 1), "gl3_delta_inner: %d tokens of %d", T, Rp);
+    if (mt == 1 || lds > 64 * 1024)
+      delta_inner_mfma_kernel<1><<<dim3(nb, (T + 15) / 16), dim3(256), (size_t)16 * (Rp + 8) * sizeof(bf16_t), stream>>>(
+          proj, (const bf16_t*)w2, A_log, dt_bias, decay, gate, s);
+    else
+      delta_inner_mfma_kernel<4><<<dim3(nb, (T + 63) / 64), dim3(256), lds, stream>>>(proj, (const bf16_t*)w2, A_log, dt_bias,
+                                                                                      decay, gate, s);
+  } else {
+    GL3_REQUIRE(false, "gl3_delta_inner: unknown dtype %d", w_dtype);
   }
   GL3_LAUNCH_CHECK();
   return 0;

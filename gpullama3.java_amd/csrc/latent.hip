@@ -16,7 +16,8 @@
 #include "common.h"
 
 // proj [T][ld] float: the query latent's sums from col_q (q_rank of them), the key/value latent's from col_kv (rank,
-// then rot). cq [T][q_rank] = proj / rms * wq. The cache row (tiles of gl3_k_offset, one head of dk elements):
+// then rot; negative: the step writes no latents, k_cache is not touched). cq [T][q_rank] = proj / rms * wq (wq null: the
+// sums as they are, queries that need no latent). The cache row (tiles of gl3_k_offset, one head of dk elements):
 // [proj / rms * wkv | the rot part turned in adjacent pairs by the token's position | zeros].
 // runs: offsets [H + 1] and sorted [T H] such that "expert" h owns the rows t * H + h of all tokens.
 template <typename TC>
@@ -31,13 +32,23 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const float* __restric
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const float* row = proj + (long)t * ld;
+  // the runs: token t writes its own places
+  for (int h = threadIdx.x; h < H; h += blockDim.x) sorted[(long)h * T + t] = t * H + h;
+  if (t == 0)
+    for (int h = threadIdx.x; h <= H; h += blockDim.x) offsets[h] = h * T;
   float sq = 0.f, sk = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) sq = fmaf(row[col_q + i], row[col_q + i], sq);
+  if (wq) {
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) sq = fmaf(row[col_q + i], row[col_q + i], sq);
+    sq = block_sum(sq, scratch);
+    const float iq = 1.0f / sqrtf(sq / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) cq[(long)t * q_rank + i] = from_f32<TC>(row[col_q + i] * iq * wq[i]);
+  } else {
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) cq[(long)t * q_rank + i] = from_f32<TC>(row[col_q + i]);
+  }
+  if (col_kv < 0) return;
   for (int i = threadIdx.x; i < rank; i += blockDim.x) sk = fmaf(row[col_kv + i], row[col_kv + i], sk);
-  sq = block_sum(sq, scratch);
   sk = block_sum(sk, scratch);
-  const float iq = 1.0f / sqrtf(sq / (float)q_rank + eps), ik = 1.0f / sqrtf(sk / (float)rank + eps);
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) cq[(long)t * q_rank + i] = from_f32<TC>(row[col_q + i] * iq * wq[i]);
+  const float ik = 1.0f / sqrtf(sk / (float)rank + eps);
   const int p = positions[t];
   const int page = block_table[(long)table_rows[t] * table_stride + p / page_size], in_page = p % page_size;
   TC* kp = k_cache + (long)page * page_size * dk;
@@ -51,10 +62,6 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const float* __restric
     kp[gl3_k_offset(in_page, rank + 2 * i + 1, dk)] = from_f32<TC>(v * c + u * s);
   }
   for (int i = rank + rot + threadIdx.x; i < dk; i += blockDim.x) kp[gl3_k_offset(in_page, i, dk)] = from_f32<TC>(0.f);
-  // the runs: token t writes its own places
-  for (int h = threadIdx.x; h < H; h += blockDim.x) sorted[(long)h * T + t] = t * H + h;
-  if (t == 0)
-    for (int h = threadIdx.x; h <= H; h += blockDim.x) offsets[h] = h * T;
 }
 
 extern "C" int gl3_latent_prep(const float* proj, long ld, int n_tokens, int col_q, int q_rank, int col_kv, int rank, int rot,
@@ -63,11 +70,11 @@ extern "C" int gl3_latent_prep(const float* proj, long ld, int n_tokens, int col
                                void* k_cache, int dtype, int page_size, int dk, int H, int* offsets, int* sorted,
                                hipStream_t stream) {
   if (n_tokens == 0) return 0;
-  GL3_REQUIRE(proj && wq && wkv && positions && table_rows && block_table && cq && k_cache && offsets && sorted,
+  GL3_REQUIRE(proj && cq && offsets && sorted && (col_kv < 0 || (wkv && positions && table_rows && block_table && k_cache)),
               "gl3_latent_prep: null argument");
   GL3_REQUIRE(n_tokens > 0 && q_rank > 0 && rank > 0 && rot >= 0 && rot % 2 == 0 && (rot == 0 || (cos_t && sin_t)) && H > 0,
               "gl3_latent_prep: latents of %d and %d, %d rotated elements", q_rank, rank, rot);
-  GL3_REQUIRE(col_q >= 0 && col_q + q_rank <= ld && col_kv >= 0 && col_kv + rank + rot <= ld, "gl3_latent_prep: columns beyond the rows");
+  GL3_REQUIRE(col_q >= 0 && col_q + q_rank <= ld && col_kv + rank + rot <= ld, "gl3_latent_prep: columns beyond the rows");
   GL3_REQUIRE(dk >= rank + rot && dk % 16 == 0 && page_size % 32 == 0 && table_stride > 0,
               "gl3_latent_prep: cached rows of %d for %d + %d elements, pages of %d", dk, rank, rot, page_size);
   GL3_REQUIRE((long)n_tokens * H < (1L << 31), "gl3_latent_prep: too many (token, head) rows");
@@ -160,7 +167,8 @@ extern "C" int gl3_sigmoid_gate(void* a, int dtype, const float* gate, long ld_g
 // shared memory ONCE for all its heads: as rows [key][dk] for the scores' operand, and the first `rank` columns
 // again transposed, [dim][key], for the second product's (the cache has no transposed copy of a latent).
 // Scores S = Q K^T with v_mfma_f32_16x16x32_bf16 (a lane ends up with 4 rows x 1 key of each 16 x 16 tile), scale,
-// causal mask by each pair's own position, running maximum and sum per row in 32-bit (reduced over the 16 lanes that
+// causal mask by each pair's own position (with a window: the keys p - window < j <= p, and the walk begins at the chunk
+// that holds the first pair's first key), running maximum and sum per row in 32-bit (reduced over the 16 lanes that
 // share a row), the weights in bfloat16 through a wave's own patch of shared memory into operand order, O += P V.
 // A decode step is the same kernel with one token a sequence (rows = heads).
 typedef __bf16 la_bf16x8 __attribute__((ext_vector_type(8)));
@@ -190,7 +198,7 @@ template <int NW, int RT, int MAXKS, int MAXDT>
 __global__ __launch_bounds__(NW * 64) void latent_attention_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_cache, const int* __restrict__ cu_seqlens,
     const int* __restrict__ kv_before, const int* __restrict__ block_table, const int* __restrict__ seq_rows, int table_stride,
-    bf16_t* __restrict__ out, long out_stride, int H, int dk, int rank, int page_size, float scale, int n_splits,
+    bf16_t* __restrict__ out, long out_stride, int H, int dk, int rank, int page_size, int window, float scale, int n_splits,
     float* __restrict__ part_o, float* __restrict__ part_ml) {
   // a wave takes RT tiles of 16 pairs: an operand of keys or values read from shared memory serves all of them
   constexpr int MAXP = (32 * MAXKS * 4 + NW * 64 - 1) / (NW * 64);      // pieces of a chunk that a thread carries
@@ -240,9 +248,11 @@ __global__ __launch_bounds__(NW * 64) void latent_attention_kernel(
   const int last = (row0 + ROWS < rows_total ? row0 + ROWS : rows_total) - 1;
   const int p_max = before + last / H;
   // this block's share of the keys: whole chunks of 32, the splits one after another
-  const int chunks = p_max / 32 + 1, per = (chunks + n_splits - 1) / n_splits;
-  const int k_lo = split * per * 32;
-  const int k_end = (split + 1) * per * 32 - 1 < p_max ? (split + 1) * per * 32 - 1 : p_max;
+  const int p_lo = window > 0 && before + row0 / H - window + 1 > 0 ? before + row0 / H - window + 1 : 0;
+  const int c_lo = p_lo / 32, chunks = p_max / 32 + 1 - c_lo, per = (chunks + n_splits - 1) / n_splits;
+  const int k_lo = (c_lo + split * per) * 32;
+  const int k_end = k_lo + per * 32 - 1 < p_max ? k_lo + per * 32 - 1 : p_max;
+  const int reach = window > 0 ? window : 0x7fffffff;
   const int cbs = dk >> 3, pieces = 32 * cbs;
   const float scale2 = scale * 1.4426950408889634f;
   // a chunk travels from memory into registers while the chunk before it is worked on; piece e is 8 consecutive
@@ -300,8 +310,9 @@ __global__ __launch_bounds__(NW * 64) void latent_attention_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         // (scores in units of ln 2: the weights are powers of two, one instruction each)
-        const float s0 = k0 + li <= pos[rt][i] ? S0[rt][i] * scale2 : -INFINITY;
-        const float s1 = k0 + 16 + li <= pos[rt][i] ? S1[rt][i] * scale2 : -INFINITY;
+        const int d0 = pos[rt][i] - (k0 + li);
+        const float s0 = d0 >= 0 && d0 < reach ? S0[rt][i] * scale2 : -INFINITY;
+        const float s1 = d0 >= 16 && d0 - 16 < reach ? S1[rt][i] * scale2 : -INFINITY;
         const float m_new = fmaxf(m_run[rt][i], la_max16(fmaxf(s0, s1)));
         const float p0 = s0 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s0 - m_new);
         const float p1 = s1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s1 - m_new);
@@ -400,8 +411,9 @@ extern "C" int gl3_latent_attention_supports(int dk, int rank, int page_size) {
 // [T H][n_splits][rank], part_ml [T H][n_splits][2] floats) a second kernel joins.
 extern "C" int gl3_latent_attention(const void* q, long q_stride, const void* k_cache, const int* cu_seqlens, const int* kv_before,
                                     const int* block_table, const int* seq_rows, int table_stride, void* out, long out_stride,
-                                    int n_tokens, int n_seqs, int max_q_len, int H, int dk, int rank, int page_size, float scale,
-                                    int n_splits, float* part_o, float* part_ml, long part_floats, hipStream_t stream) {
+                                    int n_tokens, int n_seqs, int max_q_len, int H, int dk, int rank, int page_size, int window,
+                                    float scale, int n_splits, float* part_o, float* part_ml, long part_floats,
+                                    hipStream_t stream) {
   if (n_seqs == 0 || max_q_len == 0) return 0;
   GL3_REQUIRE(q && k_cache && cu_seqlens && kv_before && block_table && out && table_stride > 0, "gl3_latent_attention: null argument");
   GL3_REQUIRE(gl3_latent_attention_supports(dk, rank, page_size),
@@ -409,7 +421,7 @@ extern "C" int gl3_latent_attention(const void* q, long q_stride, const void* k_
   GL3_REQUIRE(H > 0 && q_stride >= (long)H * dk && out_stride >= (long)H * rank && q_stride % 8 == 0 && (uintptr_t)q % 16 == 0 &&
                   (uintptr_t)k_cache % 16 == 0,
               "gl3_latent_attention: rows of %ld for %d heads of %d; queries and cache 16-byte aligned", q_stride, H, dk);
-  GL3_REQUIRE(n_splits >= 1 && n_splits <= 64, "gl3_latent_attention: n_splits=%d", n_splits);
+  GL3_REQUIRE(n_splits >= 1 && n_splits <= 64 && window >= 0, "gl3_latent_attention: n_splits=%d, window %d", n_splits, window);
   if (n_splits > 1)
     GL3_REQUIRE(part_o && part_ml && n_tokens > 0 && part_floats >= (long)n_tokens * H * n_splits * (rank + 2),
                 "gl3_latent_attention: the splits' workspace of %ld floats is too small", part_floats);
@@ -427,7 +439,7 @@ extern "C" int gl3_latent_attention(const void* q, long q_stride, const void* k_
 #define LA_GO(NW, KS, DT)                                                                                             \
   latent_attention_kernel<NW, 1, KS, DT><<<grid, dim3(NW * 64), sh, stream>>>(                                        \
       (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, cu_seqlens, kv_before, block_table, seq_rows, table_stride, \
-      (bf16_t*)out, out_stride, H, dk, rank, page_size, scale, n_splits, part_o, part_ml)
+      (bf16_t*)out, out_stride, H, dk, rank, page_size, window, scale, n_splits, part_o, part_ml)
   if (small) {
     if (nw == 4) LA_GO(4, 3, 4); else LA_GO(8, 3, 4);
   } else {

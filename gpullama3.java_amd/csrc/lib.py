@@ -69,7 +69,7 @@ def _declare(lib):
         "gl3_ssm_prep": [P, L, I, I, I, I, I, I, P, P, I, P, P, P, L, L, P, P, P, P, P, P],
         "gl3_decay_scan": [P, L, I, P, L, I, P, L, I, P, P, L, P, F, P, L, L, P, P, P, L, I, I, I, I, I, P, L, I, I, I, P],
         "gl3_group_norm_gate": [P, P, L, I, P, I, P, L, I, P, F, I, I, I, I, P, I, I, P],
-        "gl3_route": [P, I, I, I, P, P, P, P, I, I, P, F, I, P, I, P, P, I, I, F, P, P],
+        "gl3_route": [P, I, I, I, P, P, P, P, I, I, P, F, I, P, I, P, P, I, I, F, P, I, I, F, P],
         "gl3_expert_gemm": [P, I, L, I, P, I, I, I, I, P, P, I, P, I, L, I, I, I, F, F, P, P, P],
         "gl3_route_combine": [P, P, I, I, I, P, I, P, I, P, I, P, P, P, P],
         "gl3_streams_step": [P, I, I, I, P, P, P, P, P, F, P, I, P],
@@ -79,7 +79,7 @@ def _declare(lib):
         "gl3_latent_query": [P, I, I, I, I, I, P, P, P, P, I, I, P],
         "gl3_sigmoid_gate": [P, I, P, L, I, I, I, P],
         "gl3_latent_attention_supports": [I, I, I],
-        "gl3_latent_attention": [P, L, P, P, P, P, P, I, P, L, I, I, I, I, I, I, I, F, I, P, P, L, P],
+        "gl3_latent_attention": [P, L, P, P, P, P, P, I, P, L, I, I, I, I, I, I, I, I, F, I, P, P, L, P],
         "gl3_sides_norm_add": [P, P, P, P, P, F, F, I, I, P, P, P, P],
         "gl3_tanh_rows": [P, L, I, P, I, L, P],
         "gl3_mingru_scan": [P, L, I, P, L, P, P, P, I, I, I, P, P],
@@ -90,7 +90,11 @@ def _declare(lib):
         "gl3_residual_inject": [P, P, P, I, I, P],
         "gl3_delta_state_floats": [I, I, I, I, I],
         "gl3_delta_prep": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, I, L, F, F, I, P],
-        "gl3_delta_recurrence": [P, P, P, P, P, P, P, I, I, P, P, I, F, I, I, I, I, I, I, I, L, P],
+        "gl3_delta_recurrence": [P, P, P, P, P, P, P, P, I, I, P, P, I, F, I, I, I, I, I, I, I, L, I, P],
+        "gl3_delta_inner": [P, I, I, I, I, I, P, I, I, I, I, P, P, P, P, I, I, I, I, P],
+        "gl3_conv_heads": [P, I, L, P, I, P, L, L, P, P, P, P, P, P, I, P, P, I, P, P, I, F, P, P, P, I, I, I, I, I, I, I, I, P],
+        "gl3_side_gate": [P, P, I, P, L, I, P, P, L, I, I, I, I, I, I, P],
+        "gl3_norm_add_next": [P, P, P, F, I, I, P, F, P, I, P, P, P],
         "gl3_sample": [P, L, P, P, P, P, P, I, I, P, I, P],
         "gl3_sample_work_floats": [I, I],
         "gl3_argmax": [P, L, P, P, I, I, P],
@@ -816,7 +820,7 @@ ROUTE_MAX_TOP, ROUTE_MAX_EXPERTS = 16, 1024      # as csrc/routed.hip has them
 
 
 def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, correction=None, sum_eps=0.0, n_experts=None,
-          in_wts=None, gate_col=None, gate_out=None, norm=None, norm_out=None):
+          in_wts=None, gate_col=None, gate_out=None, norm=None, norm_out=None, groups=None, weight_scale=1.0):
     """Router logits [T, E] float32 -> the ``top`` largest per token (``idx`` [T, top] int32, the lower number wins a
     tie) with the softmax over them alone (``wts`` [T, top]); and the (token, choice) pairs ordered by expert:
     ``offsets`` [E + 1] int32, ``pairs`` [T top] int32 (pair t * top + j). ``always``: every token has one more pair
@@ -829,7 +833,9 @@ def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, cor
     whose sigmoid multiplies the output of the expert that every token passes: into ``wts`` where that expert has pairs
     (``always``), and to ``gate_out`` [T] where given. ``norm = (ssq, n_partials, d, eps)`` (at most 64 tokens, with
     ``in_wts``): the rows that the experts multiply lack their 1 / rms, which is made from the partial sums of squares,
-    rides in ``in_wts`` and goes to ``norm_out`` [T] where given."""
+    rides in ``in_wts`` and goes to ``norm_out`` [T] where given. ``groups = (count, keep)`` (with ``scores``): the experts
+    form ``count`` equal groups of neighbours, of which those with the ``keep`` largest choice scores stay open.
+    ``weight_scale`` multiplies the chosen experts' weights."""
     _dev(logits, "logits", torch.float32)
     T, ld = logits.shape
     E = ld if n_experts is None else int(n_experts)
@@ -858,7 +864,8 @@ def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, cor
     _check(library().gl3_route(_ptr(logits), T, E, int(top), _ptr(idx), _ptr(wts), _ptr(offsets), _ptr(pairs),
                                E if always else -1, rule, _ptr(correction), float(sum_eps), ld, _ptr(in_wts),
                                -1 if gate_col is None else int(gate_col), _ptr(gate_out), _ptr(ssq), int(n_partials), int(d),
-                               float(eps), _ptr(norm_out), _stream()), "route")
+                               float(eps), _ptr(norm_out), int(groups[0]) if groups else 1, int(groups[1]) if groups else 1,
+                               float(weight_scale), _stream()), "route")
 
 
 def expert_gemm(a, w, out, act=None, offsets=None, pairs=None, a_div=1, mfma=True, gated=None, row_in=None, row_out=None):
@@ -978,21 +985,36 @@ def latent_prep(proj, col_q, q_rank, col_kv, rank, rot, wq, wkv, eps, positions,
     first divided by its root mean square times ``wq``; the token's row of ``k_cache`` [page, 1, page_size, dk] takes
     [the second the same way with ``wkv`` | the shared part turned in adjacent pairs by the position | zeros].
     ``offsets`` [H + 1] and ``pairs`` [T H] receive the runs with which ``expert_gemm`` works head by head on rows
-    [T H, *] (row t H + h is head h of token t)."""
-    _f32_rows(proj, "proj", max(col_q + q_rank, col_kv + rank + rot))
+    [T H, *] (row t H + h is head h of token t). ``wq`` None: the first columns are queries already, taken as they are;
+    ``col_kv`` None: the step writes no latents (``wkv``, the positions and the cache are not looked at)."""
+    _f32_rows(proj, "proj", col_q + q_rank if col_kv is None else max(col_q + q_rank, col_kv + rank + rot))
     T = proj.shape[0]
-    _dev(wq, "wq", torch.float32); _dev(wkv, "wkv", torch.float32); _dev(cq, "cq"); _dev(k_cache, "k_cache", cq.dtype)
+    _dev(cq, "cq"); _dev(offsets, "offsets", torch.int32); _dev(pairs, "pairs", torch.int32)
+    if wq is not None:
+        _dev(wq, "wq", torch.float32)
+        if wq.shape != (q_rank,):
+            raise KernelError(f"latent_prep: a weight {tuple(wq.shape)} for a query latent of {q_rank}")
+    if cq.shape != (T, q_rank) or offsets.numel() != H + 1 or pairs.numel() != T * H:
+        raise KernelError(f"latent_prep: cq {tuple(cq.shape)}, {offsets.numel()} offsets, {pairs.numel()} pairs for {T} tokens of {H} heads")
+    if col_kv is None:
+        return _check(library().gl3_latent_prep(_ptr(proj), proj.stride(0), T, int(col_q), int(q_rank), -1, int(rank), 0, _ptr(wq),
+                                                c_void_p(0), float(eps), c_void_p(0), c_void_p(0), c_void_p(0), 1, c_void_p(0),
+                                                c_void_p(0), _ptr(cq), c_void_p(0), _code(cq, "cq"), 32, -(-rank // 16) * 16, int(H),
+                                                _ptr(offsets), _ptr(pairs), _stream()), "latent_prep")
+    _dev(wkv, "wkv", torch.float32); _dev(k_cache, "k_cache", cq.dtype)
     _dev(positions, "positions", torch.int32); _dev(table_rows, "table_rows", torch.int32)
     _dev(block_table, "block_table", torch.int32); _dev(offsets, "offsets", torch.int32); _dev(pairs, "pairs", torch.int32)
     if rot:
         _dev(cos, "cos", torch.float32); _dev(sin, "sin", torch.float32)
         if cos.shape != sin.shape or cos.dim() != 2 or cos.shape[1] != rot // 2:
             raise KernelError(f"latent_prep: table {tuple(cos.shape)} for {rot} rotated elements")
-    if (wq.shape != (q_rank,) or wkv.shape != (rank,) or cq.shape != (T, q_rank) or k_cache.dim() != 4 or k_cache.shape[1] != 1
+    if (wkv.shape != (rank,) or cq.shape != (T, q_rank) or k_cache.dim() != 4 or k_cache.shape[1] != 1
             or k_cache.shape[2] != page_size or positions.numel() != T or table_rows.numel() != T or block_table.dim() != 2
             or offsets.numel() != H + 1 or pairs.numel() != T * H):
-        raise KernelError(f"latent_prep: weights {tuple(wq.shape)}, {tuple(wkv.shape)}; cq {tuple(cq.shape)}; cache "
+        raise KernelError(f"latent_prep: weight {tuple(wkv.shape)}; cq {tuple(cq.shape)}; cache "
                           f"{tuple(k_cache.shape)}; {offsets.numel()} offsets, {pairs.numel()} pairs for {T} tokens of {H} heads")
+    if int(col_kv) < 0:
+        raise KernelError("latent_prep: a negative column")
     _check(library().gl3_latent_prep(_ptr(proj), proj.stride(0), T, int(col_q), int(q_rank), int(col_kv), int(rank), int(rot),
                                      _ptr(wq), _ptr(wkv), float(eps), _ptr(positions), _ptr(table_rows), _ptr(block_table),
                                      block_table.shape[1], _ptr(cos), _ptr(sin), _ptr(cq), _ptr(k_cache), _code(cq, "cq"),
@@ -1021,22 +1043,24 @@ def latent_attention_fits(dk, rank, page_size):
     return bool(library().gl3_latent_attention_supports(int(dk), int(rank), int(page_size)))
 
 
-def latent_splits(n_seqs, max_q_len, H, kv_len):
+def latent_splits(n_seqs, max_q_len, H, kv_len, window=None):
     """Blocks that share a sequence's cached rows in ``latent_attention``: a step of few (token, head) tiles over
     many keys is cut until the chip has blocks, each with at least four chunks of 32 keys."""
+    if window:      # (what the tokens of one tile of pairs can see together)
+        kv_len = min(kv_len, window + 32 + 128 // H)
     rows = max_q_len * H
     blocks = n_seqs * -(-rows // (64 if rows <= 64 else 128))      # (as the kernel's launch cuts the pairs into tiles)
     return int(max(1, min(256 // max(blocks, 1), kv_len // 128, 32)))
 
 
 def latent_attention(q, k_cache, cu_seqlens, kv_before, block_table, out, max_q_len, H, rank, scale, seq_rows=None,
-                     n_splits=1, part_o=None, part_ml=None):
+                     n_splits=1, part_o=None, part_ml=None, window=None):
     """Causal attention of ``q`` [T, H dk] (bfloat16) over a cache of one array, ``k_cache`` [page, 1, page_size, dk],
     whose rows are keys and, in their first ``rank`` elements, values, for all H heads alike; ``out`` [T, H rank].
     ``cu_seqlens`` [B + 1] and ``kv_before`` [B] say which tokens of the packed ``q`` belong to which sequence and
     where they sit in it; ``seq_rows`` [B] (optional) names each sequence's row of ``block_table``. With ``n_splits``
     > 1 (``latent_splits``) the keys are shared out over blocks whose parts go through ``part_o`` (T H n_splits rank
-    floats) and ``part_ml`` (T H n_splits 2 floats)."""
+    floats) and ``part_ml`` (T H n_splits 2 floats). ``window``: n: a query sees its own position and the n - 1 before it."""
     _dev(q, "q", torch.bfloat16, contiguous=False); _dev(out, "out", torch.bfloat16, contiguous=False)
     _dev(k_cache, "k_cache", torch.bfloat16)
     _dev(cu_seqlens, "cu_seqlens", torch.int32); _dev(kv_before, "kv_before", torch.int32)
@@ -1062,7 +1086,7 @@ def latent_attention(q, k_cache, cu_seqlens, kv_before, block_table, out, max_q_
         floats = T * H * n_splits * (rank + 2)
     _check(library().gl3_latent_attention(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(cu_seqlens), _ptr(kv_before),
                                           _ptr(block_table), _ptr(seq_rows), block_table.shape[1], _ptr(out), out.stride(0), T, B,
-                                          int(max_q_len), int(H), dk, int(rank), page, float(scale), int(n_splits),
+                                          int(max_q_len), int(H), dk, int(rank), page, int(window or 0), float(scale), int(n_splits),
                                           _ptr(part_o), _ptr(part_ml), floats, _stream()),
            "latent_attention")
 
@@ -1207,9 +1231,10 @@ def delta_state_floats(H, G, D, Dv, taps):
 
 
 def _delta_common(state, cu_seqlens, slot_ids, H, G, D, Dv, taps, who):
-    _dev(state, "state", torch.float32); _dev(cu_seqlens, "cu_seqlens", torch.int32); _dev(slot_ids, "slot_ids", torch.int32)
+    _dev(state, "state", torch.float32, contiguous=False)
+    _dev(cu_seqlens, "cu_seqlens", torch.int32); _dev(slot_ids, "slot_ids", torch.int32)
     B = slot_ids.numel()
-    if state.dim() != 2 or state.shape[1] < delta_state_floats(H, G, D, Dv, taps) or cu_seqlens.numel() != B + 1:
+    if state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < delta_state_floats(H, G, D, Dv, taps) or cu_seqlens.numel() != B + 1:
         raise KernelError(f"{who}: state {tuple(state.shape)}, {cu_seqlens.numel()} bounds for {B} sequences")
     return B
 
@@ -1219,18 +1244,26 @@ def delta_prep(proj, offsets, conv_w, A_log, dt_bias, state, cu_seqlens, seq_of_
     """The step's q, k, v after the short convolution, silu and (q, k) the scaling to unit length into ``act``
     [T, 2 G D + H Dv], the heads' decays and write strengths into ``gates`` [T, 2 H]; then each sequence's held
     inputs move on. ``proj`` [T, ld] float32; ``offsets``: the first columns of q, k, v, b and a in it.
-    ``one_token_each``: the caller vouches that every sequence brings exactly one token (one launch less)."""
+    ``one_token_each``: the caller vouches that every sequence brings exactly one token (one launch less). ``A_log`` and
+    ``dt_bias`` None: the decays are per key channel (``delta_inner``): ``gates`` takes the strengths alone, in its second
+    half, and the last of ``offsets`` is not looked at."""
     _dev(proj, "proj", torch.float32, contiguous=False)
-    for t, n in ((conv_w, "conv_w"), (A_log, "A_log"), (dt_bias, "dt_bias"), (act, "act"), (gates, "gates")):
+    for t, n in ((conv_w, "conv_w"), (act, "act"), (gates, "gates")):
         _dev(t, n, torch.float32)
+    if (A_log is None) != (dt_bias is None):
+        raise KernelError("delta_prep: the decays' numbers come together")
+    if A_log is not None:
+        _dev(A_log, "A_log", torch.float32); _dev(dt_bias, "dt_bias", torch.float32)
+        if A_log.shape != (H,) or dt_bias.shape != (H,):
+            raise KernelError(f"delta_prep: {tuple(A_log.shape)} and {tuple(dt_bias.shape)} numbers for {H} heads")
     _dev(seq_of_token, "seq_of_token", torch.int32)
     T = proj.shape[0]
     C = 2 * G * D + H * Dv
     B = _delta_common(state, cu_seqlens, slot_ids, H, G, D, Dv, taps, "delta_prep")
-    if (proj.dim() != 2 or proj.stride(1) != 1 or conv_w.shape != (C, taps) or A_log.shape != (H,) or dt_bias.shape != (H,)
+    if (proj.dim() != 2 or proj.stride(1) != 1 or conv_w.shape != (C, taps)
             or act.shape != (T, C) or gates.shape != (T, 2 * H) or seq_of_token.numel() != T or len(offsets) != 5):
         raise KernelError(f"delta_prep: proj {tuple(proj.shape)}, conv {tuple(conv_w.shape)}, act {tuple(act.shape)}")
-    ends = (G * D, G * D, H * Dv, H, H)
+    ends = (G * D, G * D, H * Dv, H, H if A_log is not None else 0)
     if any(o < 0 or o + e > proj.shape[1] for o, e in zip(offsets, ends)):
         raise KernelError(f"delta_prep: columns {tuple(offsets)} of rows of {proj.shape[1]}")
     _check(library().gl3_delta_prep(_ptr(proj), _ptr(conv_w), _ptr(A_log), _ptr(dt_bias), _ptr(state), _ptr(cu_seqlens),
@@ -1239,10 +1272,12 @@ def delta_prep(proj, offsets, conv_w, A_log, dt_bias, state, cu_seqlens, seq_of_
                                     float(q_scale), int(bool(one_token_each) and T == B), _stream()), "delta_prep")
 
 
-def delta_recurrence(act, gates, state, cu_seqlens, slot_ids, readout, proj, off_gate, norm_w, out, H, G, D, Dv, taps, eps):
+def delta_recurrence(act, gates, state, cu_seqlens, slot_ids, readout, proj, off_gate, norm_w, out, H, G, D, Dv, taps, eps,
+                     decay=None, gate_act="silu"):
     """The rule itself, token by token for every sequence of the step from the state it holds, then the read-outs'
     norm: ``out[t, h] = o[t, h] / rms * norm_w * silu(gate[t, h])`` (``out`` [T, H Dv] float32 or bfloat16), the gate in
-    columns ``off_gate`` .. of ``proj``; ``readout`` [T, H Dv] float32 is scratch for the raw read-outs."""
+    columns ``off_gate`` .. of ``proj``; ``readout`` [T, H Dv] float32 is scratch for the raw read-outs. ``decay`` [T, H D]
+    float32: a factor per key channel in place of the heads' decays; ``gate_act``: "silu" or "sigmoid"."""
     _dev(act, "act", torch.float32); _dev(gates, "gates", torch.float32); _dev(readout, "readout", torch.float32)
     _dev(proj, "proj", torch.float32, contiguous=False); _dev(norm_w, "norm_w", torch.float32); _dev(out, "out")
     T = act.shape[0]
@@ -1252,10 +1287,118 @@ def delta_recurrence(act, gates, state, cu_seqlens, slot_ids, readout, proj, off
             or proj.shape[0] != T or off_gate < 0 or off_gate + H * Dv > proj.shape[1]):
         raise KernelError(f"delta_recurrence: act {tuple(act.shape)}, gates {tuple(gates.shape)}, out {tuple(out.shape)}, "
                           f"proj {tuple(proj.shape)}")
-    _check(library().gl3_delta_recurrence(_ptr(act), _ptr(gates), _ptr(state), _ptr(cu_seqlens), _ptr(slot_ids),
+    if decay is not None:
+        _dev(decay, "decay", torch.float32)
+        if decay.shape != (T, H * D):
+            raise KernelError(f"delta_recurrence: decays {tuple(decay.shape)} for {H} heads of {D}")
+    if gate_act not in ("silu", "sigmoid"):
+        raise KernelError(f"delta_recurrence: a gate with {gate_act!r} is not built (silu, sigmoid)")
+    _check(library().gl3_delta_recurrence(_ptr(act), _ptr(gates), _ptr(decay), _ptr(state), _ptr(cu_seqlens), _ptr(slot_ids),
                                           _ptr(readout), _ptr(proj), proj.stride(0), off_gate, _ptr(norm_w), _ptr(out),
-                                          _code(out, "out"), float(eps), T, B, H, G, D, Dv, taps, state.stride(0), _stream()),
-           "delta_recurrence")
+                                          _code(out, "out"), float(eps), T, B, H, G, D, Dv, taps, state.stride(0),
+                                          int(gate_act == "sigmoid"), _stream()), "delta_recurrence")
+
+
+def delta_inner(proj, col_a, rank_a, col_g, rank_g, w2, rows_a, A_log, dt_bias, decay, gate, H, D, Dv):
+    """The second steps of a delta rule's two-step projections: ``proj`` [T, ld] float32 holds the first steps' sums
+    (``rank_a`` columns from ``col_a`` for the decays, ``rank_g`` from ``col_g`` for the gate), ``w2`` the second steps' rows,
+    the decays' first (``rows_a`` of them, of which H D count), then the gate's (of which H Dv count), both padded with zero
+    rows to multiples of 64, with zeros behind each row's numbers up to a multiple of 32. ``decay`` [T, H D] =
+    exp(-exp(A_log[h]) softplus(sum + dt_bias)), ``gate`` [T, H Dv] = the sums; both float32."""
+    _f32_rows(proj, "proj", max(col_a + rank_a, col_g + rank_g))
+    T = proj.shape[0]
+    _dev(w2, "w2")
+    for t, n in ((A_log, "A_log"), (dt_bias, "dt_bias"), (decay, "decay"), (gate, "gate")):
+        _dev(t, n, torch.float32)
+    if (w2.dim() != 2 or A_log.shape != (H,) or dt_bias.shape != (H * D,) or decay.shape != (T, H * D)
+            or gate.shape != (T, H * Dv) or not 0 < rows_a < w2.shape[0]):
+        raise KernelError(f"delta_inner: w2 {tuple(w2.shape)}, {tuple(A_log.shape)}, {tuple(dt_bias.shape)}, decay {tuple(decay.shape)}, "
+                          f"gate {tuple(gate.shape)} for {H} heads of {D} and {Dv}")
+    _check(library().gl3_delta_inner(_ptr(proj), proj.stride(0), int(col_a), int(rank_a), int(col_g), int(rank_g), _ptr(w2),
+                                     _code(w2, "w2"), w2.shape[1], int(rows_a), w2.shape[0] - int(rows_a), _ptr(A_log),
+                                     _ptr(dt_bias), _ptr(decay), _ptr(gate), T, H, D, Dv, _stream()), "delta_inner")
+
+
+def conv_heads(rows, conv_w, state, state_off, cu_seqlens, seq_of_token, slot_ids, positions, table_rows, block_table, rotation,
+               q_out, k_cache, v_cache, n_heads, n_kv, head_dim, v_head_dim, page_size, norm=None, one_token_each=False):
+    """Queries, keys and values behind a causal convolution over time, from ``rows`` [T, ld] (the stacked projection: heads
+    of ``head_dim`` for q and k, of ``v_head_dim`` for v, from column 0 on) to ``q_out`` [T, n_heads head_dim] and the paged
+    cache; then each sequence's held inputs move on. ``conv_w`` float32 [taps, channels], the last row the current token's;
+    ``state`` float32 [slots, ...] holds the last taps - 1 inputs from ``state_off`` on, [taps - 1, channels], oldest first.
+    ``rotation = (rot_dim, cos, sin)`` or None turns q and k in adjacent pairs; ``norm = (eps, dim, q_weight, k_weight)`` or
+    None then divides each head by its root mean square over its first ``dim`` elements (weights float32 [head_dim] or None).
+    ``one_token_each``: the caller vouches that every sequence brings exactly one token (one launch less)."""
+    _dev(rows, "rows", contiguous=False); _dev(conv_w, "conv_w", torch.float32)
+    _dev(q_out, "q_out", rows.dtype); _dev(k_cache, "k_cache", rows.dtype); _dev(v_cache, "v_cache", rows.dtype)
+    for t, n in ((cu_seqlens, "cu_seqlens"), (seq_of_token, "seq_of_token"), (slot_ids, "slot_ids"), (positions, "positions"),
+                 (table_rows, "table_rows"), (block_table, "block_table")):
+        _dev(t, n, torch.int32)
+    T, B = rows.shape[0], slot_ids.numel()
+    C = (n_heads + n_kv) * head_dim + n_kv * v_head_dim
+    if (rows.dim() != 2 or rows.stride(1) != 1 or rows.shape[1] < C or conv_w.dim() != 2 or conv_w.shape[1] != C
+            or q_out.shape != (T, n_heads * head_dim) or positions.numel() != T or seq_of_token.numel() != T
+            or table_rows.numel() != T or cu_seqlens.numel() != B + 1 or block_table.dim() != 2):
+        raise KernelError(f"conv_heads: rows {tuple(rows.shape)}, weights {tuple(conv_w.shape)}, q {tuple(q_out.shape)} for {C} channels "
+                          f"of {T} tokens")
+    taps = conv_w.shape[0]
+    _state_area(state, state_off, C * (taps - 1), "conv_heads")
+    _check_cache(k_cache, v_cache, n_kv, page_size, head_dim, "conv_heads", v_head_dim)
+    rot, cos, sin = rotation if rotation is not None else (0, None, None)
+    if rotation is not None:
+        _dev(cos, "cos", torch.float32); _dev(sin, "sin", torch.float32)
+        if cos.shape != sin.shape or cos.dim() != 2 or cos.shape[1] != rot // 2:
+            raise KernelError(f"conv_heads: table {tuple(cos.shape)} for {rot} rotated elements")
+    eps, dim, qw, kw = norm if norm is not None else (-1.0, head_dim, None, None)
+    for w in (qw, kw):
+        if w is not None:
+            _dev(w, "norm weight", torch.float32)
+            if w.shape != (head_dim,):
+                raise KernelError(f"conv_heads: a norm's weight {tuple(w.shape)} for heads of {head_dim}")
+    _check(library().gl3_conv_heads(_ptr(rows), _code(rows, "rows"), rows.stride(0), _ptr(conv_w), taps, _ptr(state),
+                                    state.stride(0), int(state_off), _ptr(cu_seqlens), _ptr(seq_of_token), _ptr(slot_ids),
+                                    _ptr(positions), _ptr(table_rows), _ptr(block_table), block_table.shape[1], _ptr(cos),
+                                    _ptr(sin), int(rot), _ptr(qw), _ptr(kw), int(dim), float(eps), _ptr(q_out), _ptr(k_cache),
+                                    _ptr(v_cache), T, B, n_heads, n_kv, head_dim, v_head_dim, page_size,
+                                    int(bool(one_token_each) and T == B), _stream()), "conv_heads")
+
+
+def side_gate(x, w, table, col, ids, out, act="gelu_tanh", mfma=True):
+    """``out[t, n] = act(x[t] . w[n]) * table[ids[t], col + n]`` for the rows n of ``w`` [dim, d], zeros behind them: ``x``
+    float32 [T, d], ``out`` [T, at least dim] in the type of ``w`` and ``table`` [rows, columns]."""
+    _dev(x, "x", torch.float32); _dev(w, "w"); _dev(table, "table", w.dtype); _dev(out, "out", w.dtype); _dev(ids, "ids", torch.int32)
+    T, d = x.shape
+    if w.dim() != 2 or w.shape[1] != d or table.dim() != 2 or ids.numel() != T or out.dim() != 2 or out.shape[0] != T             or out.shape[1] < w.shape[0] or col < 0 or col + w.shape[0] > table.shape[1]:
+        raise KernelError(f"side_gate: x {tuple(x.shape)}, w {tuple(w.shape)}, table {tuple(table.shape)} from {col}, out {tuple(out.shape)}")
+    if act not in ACTIVATIONS:
+        raise KernelError(f"side_gate: activation {act!r} is not built ({sorted(ACTIVATIONS)})")
+    _check(library().gl3_side_gate(_ptr(x), _ptr(w), _code(w, "w"), _ptr(table), table.stride(0), int(col), _ptr(ids), _ptr(out),
+                                   out.stride(0), out.shape[1], T, d, w.shape[0], ACTIVATIONS[act], int(bool(mfma)), _stream()),
+           "side_gate")
+
+
+def norm_add_next(x, y, w, eps, next_weight=None, next_eps=0.0, h=None, xg=None, ssq=None):
+    """``x += y / sqrt(mean(y^2) + eps) * w`` (float32 rows of a multiple of 4 elements), and of the completed rows what the
+    norm that reads them next makes: ``h`` = row / sqrt(mean(row^2) + next_eps) * next_weight in h's type, and/or ``xg``
+    bfloat16 = next_weight * row with ``ssq`` (at least 64 floats, at most 64 rows) the rows' sums of squares."""
+    _dev(x, "x", torch.float32); _dev(y, "y", torch.float32); _dev(w, "w", torch.float32)
+    if x.dim() != 2 or y.shape != x.shape or w.shape != (x.shape[1],):
+        raise KernelError(f"norm_add_next: x {tuple(x.shape)}, y {tuple(y.shape)}, weight {tuple(w.shape)}")
+    if next_weight is not None:
+        _dev(next_weight, "next_weight", torch.float32)
+        if next_weight.shape != w.shape:
+            raise KernelError(f"norm_add_next: the next norm's weight {tuple(next_weight.shape)}")
+    for t, n, dt in ((h, "h", (torch.float32, torch.bfloat16)), (xg, "xg", torch.bfloat16)):
+        if t is not None:
+            _dev(t, n, dt)
+            if t.shape != x.shape:
+                raise KernelError(f"norm_add_next: {n} {tuple(t.shape)} for rows {tuple(x.shape)}")
+    if ssq is not None:
+        _dev(ssq, "ssq", torch.float32)
+        if ssq.numel() < 64:
+            raise KernelError("norm_add_next: sums of squares need 64 floats")
+    _check(library().gl3_norm_add_next(_ptr(x), _ptr(y), _ptr(w), float(eps), x.shape[0], x.shape[1], _ptr(next_weight),
+                                       float(next_eps), _ptr(h), _code(h, "h") if h is not None else BF16, _ptr(xg), _ptr(ssq),
+                                       _stream()), "norm_add_next")
 
 
 def decode_advance(token_ids, positions, kv_before, sampled, history, step):

@@ -22,6 +22,9 @@
 // [T] where it has no pair. ssq (not null): the rows that the experts will multiply are not normed yet; [n_partials][64]
 // partial sums of squares of the residual rows (at most 64 of them), from which 1 / sqrt(sum / d + eps) is made and
 // multiplied into in_wts (for a pair whose weight is 1 too) and handed out as norm_out [T].
+// n_groups > 1 (rule 1): the experts form that many equal groups of neighbours; a group's score is the largest choice
+// score in it, and only the experts of the `keep` best groups can be chosen (the lower number wins a tie). weight_scale
+// multiplies the chosen experts' weights.
 struct RouteExtras {
   int ld;
   float* in_wts;
@@ -31,45 +34,129 @@ struct RouteExtras {
   int n_partials, d;
   float eps;
   float* norm_out;
+  int n_groups, keep;
+  float weight_scale;
 };
+
+// Rule 1 by a whole wave: lane l holds the scores of the experts l, l + 64, ...; c: this wave's share of shared memory,
+// E choice scores and n_groups group scores.
+__device__ __forceinline__ void wave_argmax(float& v, int& i) {      // the largest v, of equal ones the lowest i
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ov = __shfl_xor(v, o, 64);
+    const int oi = __shfl_xor(i, o, 64);
+    if (ov > v || (ov == v && oi < i)) {
+      v = ov;
+      i = oi;
+    }
+  }
+}
+__device__ __forceinline__ void wave_lds_order() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+__device__ __forceinline__ void route_choose_scores(const float* __restrict__ logits, int t, int E, int top, int* idx,
+                                                    float* __restrict__ wts, int always, const float* __restrict__ correction,
+                                                    float sum_eps, const RouteExtras& x, float inv_rms, float* c) {
+  const float* z = logits + (long)t * x.ld;
+  const int lane = threadIdx.x & 63, stride = top + (always >= 0 ? 1 : 0);
+  float z_max = -INFINITY, z_sum = 0.f;
+  for (int e = lane; e < E; e += 64) z_max = fmaxf(z_max, z[e]);
+  z_max = wave_max(z_max);
+  for (int e = lane; e < E; e += 64) z_sum += expf(z[e] - z_max);
+  z_sum = wave_sum(z_sum);
+  wave_lds_order();                        // (the wave's last token is done with its share)
+  for (int e = lane; e < E; e += 64) c[e] = expf(z[e] - z_max) / z_sum + (correction ? correction[e] : 0.f);
+  wave_lds_order();
+  if (x.n_groups > 1) {
+    float* gs = c + E;
+    const int per = E / x.n_groups;
+    for (int g = lane; g < x.n_groups; g += 64) {
+      float m = -INFINITY;
+      for (int i = 0; i < per; ++i) m = fmaxf(m, c[g * per + i]);
+      gs[g] = m;
+    }
+    unsigned open = 0;                     // bit i: group lane + 64 i stays open (at most 16 of them a lane)
+    for (int n = 0; n < x.keep; ++n) {
+      float v = -INFINITY;
+      int best = 0x7fffffff;
+      for (int g = lane, i = 0; g < x.n_groups; g += 64, ++i)
+        if (!(open >> i & 1u) && (best == 0x7fffffff || gs[g] > v)) {
+          v = gs[g];
+          best = g;
+        }
+      wave_argmax(v, best);
+      if (best < x.n_groups && (best & 63) == lane) open |= 1u << (best >> 6);
+    }
+    for (int g = lane, i = 0; g < x.n_groups; g += 64, ++i)
+      if (!(open >> i & 1u))
+        for (int e = 0; e < per; ++e) c[g * per + e] = -INFINITY;
+    wave_lds_order();
+  }
+  float sum = 0.f, mine = 0.f;             // lane j keeps the score of choice j
+  for (int j = 0; j < top; ++j) {
+    float v = -INFINITY;
+    int best = 0x7fffffff;
+    for (int e = lane; e < E; e += 64)
+      if (c[e] > v) {
+        v = c[e];
+        best = e;
+      }
+    wave_argmax(v, best);
+    if (best >= E) best = j;               // (no number among the scores: any expert, but one that exists)
+    const float s = expf(z[best] - z_max) / z_sum;
+    sum += s;
+    if (lane == j) {
+      mine = s;
+      idx[(long)t * stride + j] = best;
+    }
+    if ((best & 63) == lane) c[best] = -INFINITY;
+  }
+  sum += sum_eps;
+  if (lane < top) {
+    const float w = mine / sum * x.weight_scale;
+    wts[(long)t * stride + lane] = x.in_wts ? 1.0f : w;
+    if (x.in_wts) x.in_wts[(long)t * stride + lane] = w * inv_rms;
+  }
+  if (lane == 0) {
+    const float gate = x.gate_col >= 0 ? 1.0f / (1.0f + expf(-z[x.gate_col])) : 1.0f;
+    if (always >= 0) {
+      idx[(long)t * stride + top] = always;
+      wts[(long)t * stride + top] = gate;
+      if (x.in_wts) x.in_wts[(long)t * stride + top] = inv_rms;
+    }
+    if (x.gate_out) x.gate_out[t] = gate;
+    if (x.norm_out) x.norm_out[t] = inv_rms;
+  }
+}
+
+// Rules 0 and 2, a thread a token.
 __device__ __forceinline__ void route_choose(const float* __restrict__ logits, int t, int E, int top, int* idx,
-                                             float* __restrict__ wts, int always, int scores,
-                                             const float* __restrict__ correction, float sum_eps, const RouteExtras& x,
+                                             float* __restrict__ wts, int always, int scores, const RouteExtras& x,
                                              float inv_rms) {
   const float* z = logits + (long)t * x.ld;
   const int stride = top + (always >= 0 ? 1 : 0);
   int chosen[ROUTE_MAX_TOP];
   float val[ROUTE_MAX_TOP];
-  float z_max = -INFINITY, z_sum = 1.f;
-  if (scores == 1) {
-    for (int e = 0; e < E; ++e) z_max = fmaxf(z_max, z[e]);
-    z_sum = 0.f;
-    for (int e = 0; e < E; ++e) z_sum += expf(z[e] - z_max);
-  }
   for (int j = 0; j < top; ++j) {
     int best = -1;
-    float bv = -INFINITY, bs = 0.f;
+    float bv = -INFINITY;
     for (int e = 0; e < E; ++e) {
       bool taken = false;
       for (int i = 0; i < j; ++i) taken |= chosen[i] == e;
-      const float sc = scores == 1 ? expf(z[e] - z_max) / z_sum : z[e];      // (a sigmoid keeps the logits' order)
-      const float v = (scores == 1 && correction) ? sc + correction[e] : sc;
-      if (!taken && (best < 0 || v > bv)) {
+      if (!taken && (best < 0 || z[e] > bv)) {      // (a sigmoid keeps the logits' order)
         best = e;
-        bv = v;
-        bs = sc;
+        bv = z[e];
       }
     }
     chosen[j] = best;
-    val[j] = bs;
+    val[j] = bv;
   }
   float sum = 0.f;
   if (scores == 2) {
     for (int j = 0; j < top; ++j) val[j] = 1.0f / (1.0f + expf(-val[j]));
     sum = 1.f;
-  } else if (scores == 1) {
-    for (int j = 0; j < top; ++j) sum += val[j];
-    sum += sum_eps;
   } else {
     const float largest = val[0];          // (the first chosen is the largest)
     for (int j = 0; j < top; ++j) {
@@ -79,7 +166,7 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, i
   }
   for (int j = 0; j < top; ++j) {
     idx[(long)t * stride + j] = chosen[j];
-    const float w = val[j] / sum;
+    const float w = val[j] / sum * x.weight_scale;
     wts[(long)t * stride + j] = x.in_wts ? 1.0f : w;
     if (x.in_wts) x.in_wts[(long)t * stride + j] = w * inv_rms;
   }
@@ -95,9 +182,19 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, i
 
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ logits, int T, int E, int top,
                                                          int* __restrict__ idx, float* __restrict__ wts, int always, int scores,
-                                                         const float* __restrict__ correction, float sum_eps, RouteExtras x) {
+                                                         RouteExtras x) {
   const int t = blockIdx.x * 64 + threadIdx.x;
-  if (t < T) route_choose(logits, t, E, top, idx, wts, always, scores, correction, sum_eps, x, 1.0f);
+  if (t < T) route_choose(logits, t, E, top, idx, wts, always, scores, x, 1.0f);
+}
+
+// rule 1: a wave a token, four a block
+__global__ __launch_bounds__(256) void route_scores_kernel(const float* __restrict__ logits, int T, int E, int top,
+                                                           int* __restrict__ idx, float* __restrict__ wts, int always,
+                                                           const float* __restrict__ correction, float sum_eps, RouteExtras x) {
+  extern __shared__ float route_lds[];      // per wave E + n_groups
+  const int wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
+  if (t < T)
+    route_choose_scores(logits, t, E, top, idx, wts, always, correction, sum_eps, x, 1.0f, route_lds + wave * (E + x.n_groups));
 }
 
 // ----------------------------------------------------------------- pairs ordered by expert
@@ -136,7 +233,8 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
                                                           int* idx, float* __restrict__ wts,
                                                           int* __restrict__ offsets, int* __restrict__ sorted, int always,
                                                           int scores, const float* __restrict__ correction, float sum_eps,
-                                                          RouteExtras x) {
+                                                          RouteExtras x, int choosers) {
+  extern __shared__ float route_lds[];      // rule 1: E + n_groups floats for each of the `choosers` waves
   __shared__ float inv_rms[64];
   if (x.ssq) {                              // (the same for all threads) a wave a row adds up its partial sums
     for (int t = threadIdx.x >> 6; t < T; t += blockDim.x >> 6) {
@@ -147,9 +245,15 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
     }
     __syncthreads();
   }
-  if ((int)threadIdx.x < T)
-    route_choose(logits, threadIdx.x, E, top, idx, wts, always, scores, correction, sum_eps, x,
-                 x.ssq ? inv_rms[threadIdx.x] : 1.0f);
+  if (scores == 1) {
+    const int wave = threadIdx.x >> 6;
+    if (wave < choosers)
+      for (int t = wave; t < T; t += choosers)
+        route_choose_scores(logits, t, E, top, idx, wts, always, correction, sum_eps, x, x.ssq ? inv_rms[t] : 1.0f,
+                            route_lds + wave * (E + x.n_groups));
+  } else if ((int)threadIdx.x < T) {
+    route_choose(logits, threadIdx.x, E, top, idx, wts, always, scores, x, x.ssq ? inv_rms[threadIdx.x] : 1.0f);
+  }
   __threadfence_block();
   __syncthreads();
   const int more = always >= 0 ? 1 : 0;
@@ -160,8 +264,8 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
 // and wts then have top + 1 entries a token, offsets E + 2.
 extern "C" int gl3_route(const float* logits, int n_tokens, int E, int top, int* idx, float* wts, int* offsets, int* sorted,
                          int always, int scores, const float* correction, float sum_eps, int ld, float* in_wts, int gate_col,
-                         float* gate_out, const float* ssq, int n_partials, int d, float eps, float* norm_out,
-                         hipStream_t stream) {
+                         float* gate_out, const float* ssq, int n_partials, int d, float eps, float* norm_out, int n_groups,
+                         int keep, float weight_scale, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   GL3_REQUIRE(logits && idx && wts && offsets && sorted, "gl3_route: null argument");
   const int more = always >= 0 ? 1 : 0;
@@ -173,15 +277,24 @@ extern "C" int gl3_route(const float* logits, int n_tokens, int E, int top, int*
   GL3_REQUIRE(!gate_out || gate_col >= 0, "gl3_route: a gate to hand out without a column of logits for it");
   GL3_REQUIRE(!ssq || (n_tokens <= 64 && n_partials > 0 && d > 0 && in_wts),
               "gl3_route: a norm carried by the pairs' weights takes at most 64 tokens and weights on the experts' inputs");
-  const RouteExtras x{ld, in_wts, gate_col, gate_out, ssq, n_partials, d, eps, norm_out};
+  GL3_REQUIRE(n_groups >= 1 && (n_groups == 1 || (scores == 1 && E % n_groups == 0 && keep >= 1 && keep <= n_groups &&
+                                                  top <= keep * (E / n_groups))),
+              "gl3_route: the %d largest of %d experts in the best %d of %d groups", top, E, keep, n_groups);
+  const RouteExtras x{ld, in_wts, gate_col, gate_out, ssq, n_partials, d, eps, norm_out, n_groups, keep, weight_scale};
+  const size_t per_wave = (size_t)(E + n_groups) * sizeof(float);
   if (n_tokens <= 64) {
-    route_few_kernel<<<dim3(1), dim3(1024), 0, stream>>>(logits, n_tokens, E, top, idx, wts, offsets, sorted, always, scores,
-                                                         correction, sum_eps, x);
+    int choosers = (int)(40 * 1024 / per_wave);      // (beside the counters of the ordering)
+    choosers = choosers > 16 ? 16 : choosers;
+    route_few_kernel<<<dim3(1), dim3(1024), scores == 1 ? choosers * per_wave : 0, stream>>>(
+        logits, n_tokens, E, top, idx, wts, offsets, sorted, always, scores, correction, sum_eps, x, choosers);
     GL3_LAUNCH_CHECK();
     return 0;
   }
-  route_topk_kernel<<<dim3((n_tokens + 63) / 64), dim3(64), 0, stream>>>(logits, n_tokens, E, top, idx, wts, always, scores,
-                                                                                 correction, sum_eps, x);
+  if (scores == 1)
+    route_scores_kernel<<<dim3((n_tokens + 3) / 4), dim3(256), 4 * per_wave, stream>>>(logits, n_tokens, E, top, idx, wts, always,
+                                                                                     correction, sum_eps, x);
+  else
+    route_topk_kernel<<<dim3((n_tokens + 63) / 64), dim3(64), 0, stream>>>(logits, n_tokens, E, top, idx, wts, always, scores, x);
   GL3_LAUNCH_CHECK();
   route_sort_kernel<<<dim3(1), dim3(1024), 0, stream>>>(idx, n_tokens * (top + more), E + more, offsets, sorted);
   GL3_LAUNCH_CHECK();

@@ -36,7 +36,7 @@ import math
 
 import torch
 
-from ..cache import KVNeed
+from ..cache import KVNeed, StateNeed
 from ..csrc import lib as K
 from ..weights.loader import TensorSpec
 from . import ops
@@ -73,7 +73,11 @@ class GQAAttention:
             raise ValueError("an attention has a window or a chunked mask, not both")
         # (rotated values, a gate per head, a rotation with values of another size, a norm on queries and keys, several
         # score maps and a mixer that only reads run on the kernels for any sizes)
-        self.general = bool(self.value_position_spec is not None or self.gated
+        self.conv_taps = int(getattr(spec, "conv_taps", 0) or 0)
+        if self.conv_taps and (self.value_position_spec is not None or self.gated or self.diff is not None or self.reads_only
+                               or self.values_are_keys or getattr(spec, "value_mix", None) is not None):
+            raise ValueError("an attention behind short convolutions has plain keys and values of its own and no gate per head")
+        self.general = bool(self.conv_taps or self.value_position_spec is not None or self.gated
                             or (spec.position is not None and self.vd != self.hs) or self.qk_norm_eps is not None
                             or self.diff is not None or self.reads_only or self.values_are_keys)
         # (a rule on scores and outputs and values blended across layers: the same path)
@@ -96,7 +100,7 @@ class GQAAttention:
         # what turns or norms heads, or gates them as a whole, goes through the kernel that does all of these
         self.turns = bool(spec.position is not None or self.value_position_spec is not None or self.gated
                           or self.qk_norm_eps is not None)
-        if self.general and (ruled or self.mix is not None) and not self.turns and dtype == torch.bfloat16:
+        if self.general and (self.conv_taps or ((ruled or self.mix is not None) and not self.turns)) and dtype == torch.bfloat16:
             one = [n for n in K.ATTENTION_HEAD_SIZES if n >= max(self.hs, self.vd)]
             if one:
                 self.hs = self.vd = one[0]
@@ -115,6 +119,9 @@ class GQAAttention:
         self.position = build_part("position", spec.position, device=device) if spec.position is not None else None
         self.value_position = (build_part("position", self.value_position_spec, device=device)
                                if self.value_position_spec is not None else None)
+        if self.conv_taps and self.position is not None and not self.position.adjacent:
+            raise ValueError("heads behind a short convolution are rotated in adjacent pairs")
+        self.channels = (self.Hq + self.Kq) * self.hs + self.Kh * self.vd
         if self.value_position is not None and self.value_position.rot_dim > self.vd_stored:
             raise ValueError(f"values of {self.vd_stored} elements cannot be rotated over {self.value_position.rot_dim}")
         self.names = spec.names
@@ -132,7 +139,10 @@ class GQAAttention:
                 out[n["v"]] = TensorSpec((self.Kh * vd, d))
         if self.sink_name:
             out[self.sink_name] = TensorSpec((self.H,), "vector", 0.0, 1.0)
-        if self.qk_norm_eps is not None:
+        if self.conv_taps:
+            for k, c in (("q_conv", self.Hq * hs), ("k_conv", self.Kq * hs), ("v_conv", self.Kh * vd)):
+                out[n[k]] = TensorSpec((c, self.conv_taps), "matrix", 0.0, 0.5)
+        if self.qk_norm_eps is not None and "q_norm" in n:
             out[n["q_norm"]] = TensorSpec((hs,), "vector")
             if not self.reads_only:
                 out[n["k_norm"]] = TensorSpec((hs,), "vector")
@@ -236,8 +246,11 @@ class GQAAttention:
                 out = torch.zeros(self.hs, dtype=torch.float32, device=w.device)
                 out[:self.hs_stored] = w.float()
                 return out
-            self.q_norm_w = padded(weights[n["q_norm"]])
-            self.k_norm_w = padded(weights[n["k_norm"]]) if not self.reads_only else None
+            one = torch.ones(self.hs_stored, device=self.w_qkv.device)      # (a norm without a weight)
+            self.q_norm_w = padded(weights[n["q_norm"]] if "q_norm" in n else one)
+            self.k_norm_w = padded(weights[n["k_norm"]] if "k_norm" in n else one) if not self.reads_only else None
+        if self.conv_taps:      # [taps, channels], in 32-bit
+            self.conv_w = torch.cat([weights[n[k]].float() for k in ("q_conv", "k_conv", "v_conv")], dim=0).t().contiguous()
         if self.diff is not None:
             lq1, lk1, lq2, lk2 = (weights[n[k]].float() for k in ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2"))
             self.diff_lambda = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + float(self.diff.offset)
@@ -252,7 +265,7 @@ class GQAAttention:
                       keep_first=self.keep_first, v_heads=None if self.maps == 1 else self.Kh, chunk=self.chunk)
 
     def state_need(self):
-        return None
+        return StateNeed(max(-(-self.channels * (self.conv_taps - 1) // 4) * 4, 4), torch.float32) if self.conv_taps else None
 
     def forward(self, ctx, h, x, run, epilogue=ops.EPI_ADD):
         """``epilogue``: EPI_ADD adds the output into the residual rows ``x``; EPI_STORE writes it to ``x``, a float32
@@ -298,7 +311,17 @@ class GQAAttention:
             if other is None or other[2] != self.vd_stored or other[0].shape[1] != Kh * other[1]:
                 raise ValueError("an attention that blends its values finds no earlier layer's values of the same heads and size")
             blend = (other[0], other[1], self.mix_lambda)
-        if writes and not self.turns:
+        q = qkv                         # (rows that begin with the queries)
+        if self.conv_taps:
+            if not writes:
+                raise ValueError("an attention behind short convolutions keeps keys and values of its own")
+            q = ctx.buffer("conv_q", (T, qn), self.dtype)
+            K.conv_heads(qkv, self.conv_w, ctx.slot_state(run.entry), 0, ctx.cu_seqlens, ctx.seq_of_token, ctx.slot_ids, ctx.positions,
+                         ops._table_rows(ctx), table, qk if pos is not None else None, q, k_cache, v_cache, Hq, Kh, hs, vd,
+                         k_cache.shape[2], norm=(self.qk_norm_eps, self.hs_stored, self.q_norm_w if "q_norm" in self.names else None,
+                                                 self.k_norm_w if "k_norm" in self.names else None) if normed else None,
+                         one_token_each=bool(ctx.decode and ctx.max_q_len == 1))
+        elif writes and not self.turns:
             K.kv_write(qkv, qn, qn + kn, ctx.positions, ops._table_rows(ctx), table, k_cache, v_cache, Kh, hs, vd,
                        k_cache.shape[2], blend=blend)
         elif blend is not None:
@@ -316,7 +339,7 @@ class GQAAttention:
         if self.diff is not None and ops.attention_kernel(ctx, self.dtype, k_cache.shape[2], Hq, Kq, hs, self.scale, vd) == "generic":
             att_dtype = torch.float32      # the maps' outputs stay in 32-bit up to their difference, where the kernel can write them so
         att = ctx.buffer("attn_out", (T, Hq * vd), att_dtype)
-        ops.attention(ctx, qkv, k_cache, v_cache, table, att, Hq, Kq, hs, self.window, self.scale, v_head_dim=vd,
+        ops.attention(ctx, q, k_cache, v_cache, table, att, Hq, Kq, hs, self.window, self.scale, v_head_dim=vd,
                       slopes=self.slopes, sink=self.sink, keep_first=self.keep_first, chunk=self.chunk,
                       n_v_heads=Kh if self.maps > 1 else None, rule=self._score_rule(qkv, qn + kn + vn))
         if self.diff is not None:
@@ -366,7 +389,9 @@ class _PaddedHeads:
         p, n, w = self.part, self.part.names, self.weights[name]
         heads = {n["q"]: (p.Hq, p.hs_stored, p.hs), n.get("k"): (p.Kq, p.hs_stored, p.hs), n.get("v"): (p.Kh, p.vd_stored, p.vd),
                  n.get("q_bias"): (p.Hq, p.hs_stored, p.hs), n.get("k_bias"): (p.Kq, p.hs_stored, p.hs),
-                 n.get("v_bias"): (p.Kh, p.vd_stored, p.vd), n.get("gate"): (p.H, p.vd_stored, p.vd)}
+                 n.get("v_bias"): (p.Kh, p.vd_stored, p.vd), n.get("gate"): (p.H, p.vd_stored, p.vd),
+                 n.get("q_conv"): (p.Hq, p.hs_stored, p.hs), n.get("k_conv"): (p.Kq, p.hs_stored, p.hs),
+                 n.get("v_conv"): (p.Kh, p.vd_stored, p.vd)}
         if name in heads and w.shape[0] == heads[name][0] * heads[name][1]:
             H, d_in, d_out = heads[name]
             out = torch.zeros((H, d_out) + tuple(w.shape[1:]), dtype=w.dtype, device=w.device)

@@ -12,6 +12,7 @@ Norm:         ``__call__(ctx, x[T,d] float32, rows=None) -> [R,d]`` in the activ
 Mixer:        ``forward(ctx, h[T,d], x[T,d] float32, run)`` adds its output into ``x``;
               ``kv_need()`` / ``state_need()`` tell the cache what one run-order entry stores.
 FeedForward:  ``forward(ctx, h[T,d], x[T,d] float32)`` adds its output into ``x``.
+Side:         ``forward(ctx, x[T,d] float32, norm_after=None)`` adds something of its own into ``x`` behind a block's sublayers.
 Position:     built by the mixer that uses it from its description (``build_part("position", ...)``).
 Block:        ``parts()`` and ``forward(ctx, x, run)``; owns the arrangement of norm, mixer and
               feed-forward. Optional: ``cache_needs() -> (KVNeed | None, StateNeed | None)`` (else the
@@ -30,7 +31,7 @@ from __future__ import annotations
 from dataclasses import dataclass
 from typing import Optional
 
-_REGISTRY = {"norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}}
+_REGISTRY = {"norm": {}, "mixer": {}, "ffn": {}, "position": {}, "block": {}, "side": {}}
 
 
 def register_part(category, kind, cls):

@@ -13,15 +13,22 @@ from . import ops
 from .base import build_part, register_part
 
 
+def _side(spec, dtype, device):
+    """What stands behind the sublayers, if the description names something."""
+    s = getattr(spec, "side", None)
+    return build_part("side", s, dtype=dtype, device=device) if s is not None else None
+
+
 class PreNormBlock:
     def __init__(self, spec, dtype, device):
+        self.side = _side(spec, dtype, device)
         self.mixer_norm = build_part("norm", spec.mixer_norm, dtype=dtype)
         self.mixer = build_part("mixer", spec.mixer, dtype=dtype, device=device)
         self.ffn_norm = build_part("norm", spec.ffn_norm, dtype=dtype) if spec.ffn is not None else None
         self.ffn = build_part("ffn", spec.ffn, dtype=dtype, device=device) if spec.ffn is not None else None
 
     def parts(self):
-        return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn) if p is not None]
+        return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn, self.side) if p is not None]
 
     def cache_needs(self):
         return self.mixer.kv_need(), self.mixer.state_need()
@@ -32,6 +39,7 @@ class PreNormBlock:
 
     def forward(self, ctx, x, run, norm_after=None):
         """``norm_after``: the norm that reads the residual rows after this block, if known."""
+        behind, norm_after = norm_after, (norm_after if self.side is None else None)
         h = self._whole_rows_for(self.mixer_norm, "takes_slices", ctx, x)(ctx, x)
         ctx.next_norm = self.ffn_norm if self.ffn is not None else norm_after
         self._whole_rows_for(self.mixer, "adds_only", ctx, x).forward(ctx, h, x, run)
@@ -40,6 +48,8 @@ class PreNormBlock:
             ctx.next_norm = norm_after
             self._whole_rows_for(self.ffn, "adds_only", ctx, x).forward(ctx, h, x)
         ctx.next_norm = None
+        if self.side is not None:
+            self.side.forward(ctx, x, behind)
 
     @staticmethod
     def _whole_rows_for(part, declares, ctx, x):
@@ -54,18 +64,19 @@ class PreNormBlock:
 
 class ParallelBlock:
     """One norm whose output feeds both the mixer and the feed-forward; both add into the residual rows:
-    ``h = norm(x); x += mixer(h) + ffn(h)``. The rows are complete after the later of the two, so only that one may
-    leave what the norm that reads them next would use."""
+    ``h = norm(x); x += mixer(h) + ffn(h)``. The rows are complete after the later of the two (or after what stands behind
+    both: ``side``), so only that one may leave what the norm that reads them next would use."""
 
     def __init__(self, spec, dtype, device):
         if spec.ffn_norm is not None:
             raise ValueError("a parallel block has one norm: its description names no norm for the feed-forward")
         self.norm = build_part("norm", spec.mixer_norm, dtype=dtype)
+        self.side = _side(spec, dtype, device)
         self.mixer = build_part("mixer", spec.mixer, dtype=dtype, device=device)
         self.ffn = build_part("ffn", spec.ffn, dtype=dtype, device=device) if spec.ffn is not None else None
 
     def parts(self):
-        return [p for p in (self.norm, self.mixer, self.ffn) if p is not None]
+        return [p for p in (self.norm, self.mixer, self.ffn, self.side) if p is not None]
 
     def cache_needs(self):
         return self.mixer.kv_need(), self.mixer.state_need()
@@ -74,6 +85,7 @@ class ParallelBlock:
         return self.norm
 
     def forward(self, ctx, x, run, norm_after=None):
+        behind, norm_after = norm_after, (norm_after if self.side is None else None)
         h = PreNormBlock._whole_rows_for(self.norm, "takes_slices", ctx, x)(ctx, x)
         if self.ffn is not None and isinstance(h, ops.Normed) and not getattr(self.ffn, "folds_norm", lambda h: False)(h):
             # a norm that a product was to take over is worked out from the rows when somebody asks for it; a
@@ -87,6 +99,8 @@ class ParallelBlock:
             ctx.next_norm = norm_after
             PreNormBlock._whole_rows_for(self.ffn, "adds_only", ctx, x).forward(ctx, h, x)
         ctx.next_norm = None
+        if self.side is not None:
+            self.side.forward(ctx, x, behind)
 
 
 class OutNormBlock:

@@ -87,6 +87,8 @@ class DecoderModel:
         self.without = ops.switches(without)
         self.blocks = [build_part("block", b, dtype=dtype, device=device) for b in spec.layers]
         self.final_norm = build_part("norm", spec.final_norm, dtype=dtype) if spec.final_norm is not None else None
+        if self.final_norm is not None:
+            self.final_norm.reads_wanted_rows = True
         # (a layer whose queries read another entry's keys and values needs the q rows alone: then stacked rows keep
         # their stored order)
         may_hold_once = not any(r.reads is not None for r in spec.run_order)
@@ -173,7 +175,7 @@ class DecoderModel:
         """Logits ``[len(want_rows), vocab]`` float32 at the wanted packed rows."""
         S = int(getattr(self.spec, "streams", 1) or 1)      # copies of the residual row per token
         x = ctx.buffer("residual", (ctx.n_tokens, self.spec.hidden), torch.float32)
-        ctx.ssq = ctx.pending = ctx.next_norm = None   # a context may run more than one forward pass: nothing is left over
+        ctx.ssq = ctx.normed = ctx.pending = ctx.next_norm = None   # a context may run more than one forward pass: nothing is left over
         ctx.token_facts, ctx.token_tables = {}, {}
         ctx.first_values = None         # (the values that later layers of a step blend into theirs, once a layer hands them out)
         ctx.rows_as_input = None        # (the address of rows whose copy in the activations' type a block has left)

@@ -38,6 +38,9 @@ class RMSNorm:
     def __call__(self, ctx, x, rows=None, name="normed"):
         """The normalised rows, or a ``Normed`` when the next product can do the work itself (few
         rows, and the kernel that last wrote exactly this tensor prepared the rows for this norm)."""
+        made = getattr(ctx, "normed", None)
+        if made is not None and made[0] == x.data_ptr() and made[1] is self and rows is None and made[2].shape == x.shape:
+            return made[2]                # (the kernel that completed the rows has made them already)
         rec = getattr(ctx, "ssq", None)
         if (getattr(ctx, "fuse", False) and rec is not None and rec[0] == x.data_ptr() and rec[4] is self
                 and x.shape[0] <= ops.FUSE_ROWS and self.dtype == torch.bfloat16):

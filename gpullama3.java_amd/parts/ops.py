@@ -168,6 +168,22 @@ def residual_written(ctx, x, ssq=None, n_partials=0, xg=None, norm=None):
     nothing."""
     if ctx is not None:
         ctx.ssq = (x.data_ptr(), ssq, n_partials, xg, norm) if ssq is not None and xg is not None else None
+        ctx.normed = None
+
+
+def normed_ahead(ctx, norm, x):
+    """A buffer for the output of ``norm`` over the residual rows ``x`` if the kernel that completes the rows may make it:
+    an RMS norm that reads every row next (not the head's, which reads wanted rows), else None. The caller says
+    ``normed_is_ready`` once the kernel has run."""
+    w = getattr(norm, "weight_f32", None)
+    if (norm is None or w is None or w.shape != (x.shape[1],) or not getattr(norm, "folds", False)
+            or getattr(norm, "reads_wanted_rows", False) or "fused" in _off(ctx)):
+        return None
+    return ctx.buffer("normed", tuple(x.shape), norm.dtype)
+
+
+def normed_is_ready(ctx, x, norm, out):
+    ctx.normed = (x.data_ptr(), norm, out)
 
 
 def _next_norm(ctx, N):

@@ -15,7 +15,8 @@ What a description may change: gated experts (``ExpertSpec.gated``: gate and up 
 grouped product's epilogue finds a gate value and its up value in neighbouring lanes and writes
 ``act(min(gate, limit)) * (clamp(up) + shift)`` directly); the other rule for choice and weights (``weights =
 "scores"``: a softmax over all router outputs, the choice by score plus a stored correction, the weights from the
-chosen scores over their sum); the third (``weights = "sigmoid"``: the largest router outputs, each weighted with
+chosen scores over their sum; ``groups``: only experts of the best groups of neighbours can be chosen; ``weight_scale``: a
+constant on the chosen experts' weights); the third (``weights = "sigmoid"``: the largest router outputs, each weighted with
 its own sigmoid); a weight that multiplies the expert's input instead of its output (``weight_on``: up and gate rows are
 linear, so the factor goes onto a pair's sums in front of the activation); a shared expert whose output is multiplied
 by a sigmoid of its own (``shared_weight``: one more row of the router's product); and identity experts
@@ -60,6 +61,12 @@ class RoutedFeedForward:
         if self.on_input and self.I:
             raise ValueError("an identity expert has no input that a weight could multiply")
         self.sum_eps = float(getattr(spec, "sum_eps", 0.0))
+        self.groups = getattr(spec, "groups", None)
+        self.weight_scale = float(getattr(spec, "weight_scale", 1.0))
+        if self.groups is not None:
+            count, keep = self.groups
+            if self.scores is not True or self.I or self.E % count or not 1 <= keep <= count or self.top > keep * (self.E // count):
+                raise ValueError(f"the {self.top} largest of the best {keep} of {count} groups of {self.E} experts")
         if not 1 <= self.top <= self.E + self.I:
             raise ValueError(f"the {self.top} largest of {self.E + self.I} experts")
         for e in (spec.expert, spec.shared):
@@ -185,7 +192,8 @@ class RoutedFeedForward:
         s_in = ctx.buffer("shared_input_weights", (T,), torch.float32) if apart and norm is not None else None
         K.route(logits, top, idx, wts, offsets, pairs, always=self.merged, scores=self.scores,
                 correction=self.correction, sum_eps=self.sum_eps, n_experts=routed, in_wts=in_wts,
-                gate_col=routed if self.shared_gated else None, gate_out=s_out, norm=norm, norm_out=s_in)
+                gate_col=routed if self.shared_gated else None, gate_out=s_out, norm=norm, norm_out=s_in,
+                groups=self.groups, weight_scale=self.weight_scale)
         row_in = in_wts.view(-1) if in_wts is not None else None
         act, gated = self._rule(self.spec.expert)
         hidden = ctx.buffer("experts_hidden", (T * per, F), self.dtype)
