@@ -38,6 +38,11 @@ layer has 8 gated experts of a quarter of that size and 2 identity experts, two 
 ``--arch lusalix`` does the same for a Lusalix model (in every layer an attention without a rotation: the shape's heads, a
 temperature on the queries, a soft cap, a distance bias, a window, a gate per element, values blended with the first
 layer's; 8 gated experts of a quarter of the shape's feed-forward size, two a token, beside a shared expert).
+``--arch banazen`` does the same for a Banazen model (layers in turns of three: an attention with the shape's heads behind
+short convolutions beside a gated delta rule with as many heads and a decay per key channel, a windowed attention over
+cached latents, and one more over the second's latents; the first layer's feed-forward is the shape's own, every other layer
+has 8 bounded experts of a quarter of that size, two a token from the best groups, beside a shared expert; a side row of 64
+elements a token and layer).
 ``--beside nolatar`` (or any of the others) puts a model of that design and the same sizes beside it instead of the Llama
 layers.
 """
@@ -124,10 +129,10 @@ def main():
     ap.add_argument("--points", default="1,64", help="further decode batch sizes, comma-separated")
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--workload", default="decode", choices=["decode", "unequal8"])
-    ap.add_argument("--arch", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex", "lusalix"],
-                    help="melizen, nodupel, nolatar, dotanex, lusalix: a model of that design with the shape's sizes beside Llama layers of "
+    ap.add_argument("--arch", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex", "lusalix", "banazen"],
+                    help="melizen, nodupel, nolatar, dotanex, lusalix, banazen: a model of that design with the shape's sizes beside Llama layers of "
                          "equal size (a line of its own form)")
-    ap.add_argument("--beside", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex"],
+    ap.add_argument("--beside", default="llama", choices=["llama", "melizen", "nodupel", "nolatar", "dotanex", "lusalix"],
                     help="with --arch: the model of equal size that is measured beside it")
     ap.add_argument("--without", default="", help="names of fast paths to switch off for a comparison on the same machine, "
                     "comma-separated (parts/ops.py: tiled, packed, fused, wide, ...); the line then says so in `config`")
@@ -432,6 +437,30 @@ def lusalix_config(shape, layers, window=1024):
             "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp} for _ in range(layers)]}
 
 
+def banazen_config(shape, layers, window=1024, side=64, inner=64):
+    """A Banazen model with the sizes of a Llama shape, layers in turns of three: an attention with the shape's heads behind
+    convolutions of 4 taps beside a delta rule with as many value heads of the same size over the shape's kv heads; an
+    attention over cached latents (the shape's heads, latents of 256 elements or four heads' size where that is less) with a
+    window; and one more that reads the second's latents. The first layer has the shape's feed-forward; every other layer 8
+    bounded experts of a quarter of its size in four groups of which three stay open, two a token, and a shared expert of
+    that size. Every token has a side row of 64 elements a layer."""
+    d, F = shape["hidden_size"], shape["intermediate_size"]
+    H, G, hs = shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
+    moe = {"kind": "moe", "router": {"experts": 8, "top": 2, "scale": 1.0, "groups": {"count": 4, "keep": 3}},
+           "expert": {"ff": F // 4, "limit": 7.0}, "shared": {"ff": F // 4, "limit": 7.0}}
+    heads = {"heads": H, "kv_heads": G, "dim": hs, "vdim": hs, "conv": 4}
+    sides = {"left": {**heads, "scale": hs ** -0.5, "rot": {"base": shape.get("rope_theta", 500000.0), "dims": hs}}, "right": heads}
+    latent = {"heads": H, "dim": hs, "vdim": hs, "kv_rank": min(4 * hs, 256), "scale": hs ** -0.5, "mask": {"size": window}}
+    out = []
+    for i in range(layers):
+        mixer = [sides, latent, {**latent, "kv_from": i - 1}][i % 3]
+        out.append({"type": "latent_attention" if i % 3 else "parallel", "mixer": mixer,
+                    "mlp": {"kind": "dense", "ff": F} if i == 0 else moe})
+    return {"architecture": "Banazen", "vocab": shape["vocab_size"], "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+            "logit_scale": 1.0, "token_side": {"dim": side}, "inner_sizes": [[inner, inner]] * layers,
+            "max_positions": shape["max_position_embeddings"], "layers": out}
+
+
 def other_beside_llama(args):
     """Prefill of one prompt and decode steps at --batch for a model of another design (--arch) and for Llama layers
     of equal size, one after the other on the same machine."""
@@ -448,7 +477,7 @@ def other_beside_llama(args):
     short = "bf16" if args.dtype == "bfloat16" else "fp32"
     arch = args.arch
     makers = {"melizen": melizen_config, "nodupel": nodupel_config, "nolatar": nolatar_config, "dotanex": dotanex_config,
-              "lusalix": lusalix_config}
+              "lusalix": lusalix_config, "banazen": banazen_config}
     beside = "llama" if args.beside == arch else args.beside
     configs = {arch: g.config_from_dict(makers[arch](shape, layers)),
                beside: g.config_from_dict({**shape, "num_hidden_layers": layers} if beside == "llama"

@@ -43,41 +43,75 @@ __device__ __forceinline__ void store8(T* __restrict__ p, const float (&in)[8]) 
   }
 }
 
-// The sums of the 8 channels from c on for token t of a sequence whose first token of this step is `first`.
-template <typename T>
-__device__ __forceinline__ void conv8(const T* __restrict__ rows, const float* __restrict__ w, const float* __restrict__ held,
-                                      const ConvHeads& s, int C, int c, int t, int first, float (&y)[8]) {
+// The sums of the 8 channels from c on for token t of a sequence whose first token of this step is `first`. TAPS: the taps,
+// 0 where only the launch knows them. The usual cases ask for everything at once, without a condition in between: a token
+// whose whole reach lies in this step, and a sequence's first token of the step, whose earlier inputs the slot holds (with
+// `move` these then move on: the sequence brings this one token, and nobody else reads these channels).
+template <typename T, int TAPS>
+__device__ __forceinline__ void conv8(const T* __restrict__ rows, const float* __restrict__ w, float* __restrict__ held,
+                                      const ConvHeads& s, int C, int c, int t, int first, bool move, float (&y)[8]) {
+  const int taps = TAPS ? TAPS : s.taps;
+  constexpr int N = TAPS ? TAPS : 1;
 #pragma unroll
   for (int e = 0; e < 8; ++e) y[e] = 0.f;
-  for (int j = 0; j < s.taps; ++j) {
-    const int src = t - (s.taps - 1) + j;
+  if (TAPS && t - first >= taps - 1) {
+    float u[N][8], f[N][8];
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      load8<T>(rows + (long)(t - (N - 1) + j) * s.ld + c, u[j]);
+      load8<float>(w + (long)j * C + c, f[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < N; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] = fmaf(f[j][e], u[j][e], y[e]);
+    return;
+  }
+  if (TAPS && t == first) {
+    float u[N][8], f[N][8];
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      if (j + 1 < N) load8<float>(held + (long)j * C + c, u[j]);
+      else load8<T>(rows + (long)t * s.ld + c, u[j]);
+      load8<float>(w + (long)j * C + c, f[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < N; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] = fmaf(f[j][e], u[j][e], y[e]);
+    if (move) {
+#pragma unroll
+      for (int j = 1; j < N; ++j) store8<float>(held + (long)(j - 1) * C + c, u[j]);
+    }
+    return;
+  }
+  for (int j = 0; j < taps; ++j) {
+    const int src = t - (taps - 1) + j;
     float u[8], f[8];
     if (src >= first) load8<T>(rows + (long)src * s.ld + c, u);
-    else load8<float>(held + (long)(src - first + s.taps - 1) * C + c, u);
+    else load8<float>(held + (long)(src - first + taps - 1) * C + c, u);
     load8<float>(w + (long)j * C + c, f);
 #pragma unroll
     for (int e = 0; e < 8; ++e) y[e] = fmaf(f[e], u[e], y[e]);
   }
-}
-
-// (every sequence brings one token: the thread that made a channel's sum is the only reader of its held inputs)
-template <typename T>
-__device__ __forceinline__ void move_on(const T* __restrict__ rows, float* __restrict__ held, const ConvHeads& s, int C, int c, int t) {
-  float u[8];
-  for (int j = 0; j + 2 < s.taps; ++j) {
-    load8<float>(held + (long)(j + 1) * C + c, u);
-    store8<float>(held + (long)j * C + c, u);
-  }
-  if (s.taps > 1) {
-    load8<T>(rows + (long)t * s.ld + c, u);
-    store8<float>(held + (long)(s.taps - 2) * C + c, u);
+  if (move) {
+    float u[8];
+    for (int j = 0; j + 2 < taps; ++j) {
+      load8<float>(held + (long)(j + 1) * C + c, u);
+      store8<float>(held + (long)j * C + c, u);
+    }
+    if (taps > 1) {
+      load8<T>(rows + (long)t * s.ld + c, u);
+      store8<float>(held + (long)(taps - 2) * C + c, u);
+    }
   }
 }
 
-// A block a token (an XCD a stretch of tokens). A query or key head takes `lp` lanes side by side, a power of two, 8
+// A block a token (an XCD a stretch of tokens), or in a step of few tokens several: grid y, of which the last makes the
+// values and the others the queries and keys. A query or key head takes `lp` lanes side by side, a power of two, 8
 // channels each; the block whose token begins a group of 8 positions (or its sequence's tokens of this step) makes the
 // values of the whole group, which lie together in the cache.
-template <typename T>
+template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void conv_heads_kernel(
     const T* __restrict__ rows, const float* __restrict__ w, float* __restrict__ state, const int* __restrict__ cu_seqlens,
     const int* __restrict__ seq_of_token, const int* __restrict__ slot_ids, const int* __restrict__ positions,
@@ -94,39 +128,42 @@ __global__ __launch_bounds__(256) void conv_heads_kernel(
   const int QK = (s.Hq + s.Kh) * s.hs, C = QK + s.Kh * s.vd, half = s.rot / 2;
   float* held = state + (long)slot_ids[b] * s.state_stride + s.held_off;
   const int heads = s.Hq + s.Kh, lanes = heads * lp;
-  for (int i0 = 0; i0 < lanes; i0 += 256) {                 // (whole waves: the sum over a head's lanes is theirs together)
-    const int i = i0 + threadIdx.x, head = i / lp, e0 = (i % lp) * 8;
-    const bool here = i < lanes && e0 < s.hs;
-    const int c = here ? head * s.hs + e0 : 0;
-    float y[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (here) conv8<T>(rows, w, held, s, C, c, t, first, y);
-    if (cos_t && here && e0 < s.rot) {
+  const int parts = gridDim.y, qk_parts = parts > 1 ? parts - 1 : 1;
+  if ((int)blockIdx.y < qk_parts) {
+    for (int i0 = 256 * blockIdx.y; i0 < lanes; i0 += 256 * qk_parts) {      // (whole waves: the sum over a head's lanes is theirs together)
+      const int i = i0 + threadIdx.x, head = i / lp, e0 = (i % lp) * 8;
+      const bool here = i < lanes && e0 < s.hs;
+      const int c = here ? head * s.hs + e0 : 0;
+      float y[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (here) conv8<T, TAPS>(rows, w, held, s, C, c, t, first, s.one_each, y);
+      if (cos_t && here && e0 < s.rot) {
 #pragma unroll
-      for (int a = 0; a < 4; ++a) {
-        const int p = e0 / 2 + a;
-        if (p < half) {
-          const float cs = cos_t[(long)pos * half + p], sn = sin_t[(long)pos * half + p];
-          const float u = y[2 * a], v = y[2 * a + 1];
-          y[2 * a] = u * cs - v * sn;
-          y[2 * a + 1] = v * cs + u * sn;
+        for (int a = 0; a < 4; ++a) {
+          const int p = e0 / 2 + a;
+          if (p < half) {
+            const float cs = cos_t[(long)pos * half + p], sn = sin_t[(long)pos * half + p];
+            const float u = y[2 * a], v = y[2 * a + 1];
+            y[2 * a] = u * cs - v * sn;
+            y[2 * a + 1] = v * cs + u * sn;
+          }
         }
       }
-    }
-    if (s.eps >= 0.f) {
-      float ss = 0.f;
+      if (s.eps >= 0.f) {
+        float ss = 0.f;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) ss = fmaf(y[e], y[e], ss);
-      for (int o = 1; o < lp; o <<= 1) ss += __shfl_xor(ss, o, 64);
-      const float inv = 1.0f / sqrtf(ss / (float)s.norm_dim + s.eps);
-      const float* nw = head < s.Hq ? qw : kw;
+        for (int e = 0; e < 8; ++e) ss = fmaf(y[e], y[e], ss);
+        for (int o = 1; o < lp; o <<= 1) ss += __shfl_xor(ss, o, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)s.norm_dim + s.eps);
+        const float* nw = head < s.Hq ? qw : kw;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) y[e] *= nw && here ? inv * nw[e0 + e] : inv;
+        for (int e = 0; e < 8; ++e) y[e] *= nw && here ? inv * nw[e0 + e] : inv;
+      }
+      if (here) {
+        if (head < s.Hq) store8<T>(q_out + (long)t * s.Hq * s.hs + c, y);
+        else store8<T>(k_cache + (page * s.Kh + head - s.Hq) * (long)s.page_size * s.hs + gl3_k_offset(in_page, e0, s.hs), y);
+      }
     }
-    if (here) {
-      if (head < s.Hq) store8<T>(q_out + (long)t * s.Hq * s.hs + c, y);
-      else store8<T>(k_cache + (page * s.Kh + head - s.Hq) * (long)s.page_size * s.hs + gl3_k_offset(in_page, e0, s.hs), y);
-      if (s.one_each) move_on<T>(rows, held, s, C, c, t);
-    }
+    if (parts > 1) return;
   }
   int run = 0;                                             // how many tokens' values this block makes
   if ((pos & 7) == 0 || t == first) {
@@ -143,7 +180,7 @@ __global__ __launch_bounds__(256) void conv_heads_kernel(
 #pragma unroll
       for (int r = 0; r < 8; ++r) {
         float y[8];
-        conv8<T>(rows, w, held, s, C, c, t + r, first, y);
+        conv8<T, TAPS>(rows, w, held, s, C, c, t + r, first, false, y);
 #pragma unroll
         for (int e = 0; e < 8; ++e) all[e][r] = from_f32<T>(y[e]);
       }
@@ -155,14 +192,13 @@ __global__ __launch_bounds__(256) void conv_heads_kernel(
         store8<T>(at + 8 * e, o);
       }
     } else {
-      for (int r = 0; r < run; ++r) {
+      for (int r = 0; r < run; ++r) {                      // (one_each: run is 1)
         float y[8];
-        conv8<T>(rows, w, held, s, C, c, t + r, first, y);
+        conv8<T, TAPS>(rows, w, held, s, C, c, t + r, first, s.one_each, y);
 #pragma unroll
         for (int e = 0; e < 8; ++e) at[8 * e + r] = from_f32<T>(y[e]);
       }
     }
-    if (s.one_each) move_on<T>(rows, held, s, C, c, t);
   }
 }
 
@@ -209,12 +245,18 @@ extern "C" int gl3_conv_heads(const void* rows, int dtype, long ld, const float*
   while (lp * 8 < hs) lp *= 2;
   const ConvHeads s{Hq, Kh, hs, vd, taps, cos_t ? rot : 0, norm_dim, ld, state_stride, held_off, eps, table_stride, page_size,
                     n_tokens, one_each};
-  const dim3 grid((unsigned)((n_tokens + 7) / 8 * 8)), block(256), sgrid(n_seqs, (unsigned)((C + 255) / 256));
+  const unsigned parts = n_tokens <= 64 ? (unsigned)(((Hq + Kh) * lp + 255) / 256 + 1) : 1;
+  const dim3 grid((unsigned)((n_tokens + 7) / 8 * 8), parts), block(256), sgrid(n_seqs, (unsigned)((C + 255) / 256));
+#define CH_TAPS(T, TAPS)                                                                                                     \
+  conv_heads_kernel<T, TAPS><<<grid, block, 0, stream>>>((const T*)rows, w, state, cu_seqlens, seq_of_token, slot_ids,       \
+                                                         positions, table_rows, block_table, cos_t, sin_t, qw, kw, (T*)q_out, \
+                                                         (T*)k_cache, (T*)v_cache, s, lp)
 #define CH_GO(T)                                                                                                              \
   do {                                                                                                                        \
-    conv_heads_kernel<T><<<grid, block, 0, stream>>>((const T*)rows, w, state, cu_seqlens, seq_of_token, slot_ids, positions, \
-                                                     table_rows, block_table, cos_t, sin_t, qw, kw, (T*)q_out, (T*)k_cache,   \
-                                                     (T*)v_cache, s, lp);                                                     \
+    if (taps == 2) CH_TAPS(T, 2);                                                                                             \
+    else if (taps == 3) CH_TAPS(T, 3);                                                                                        \
+    else if (taps == 4) CH_TAPS(T, 4);                                                                                        \
+    else CH_TAPS(T, 0);                                                                                                       \
     if (taps > 1 && !one_each) {                                                                                              \
       GL3_LAUNCH_CHECK();                                                                                                     \
       conv_heads_state_kernel<T><<<sgrid, block, 0, stream>>>((const T*)rows, state, cu_seqlens, slot_ids, s, (int)C);        \
@@ -224,6 +266,7 @@ extern "C" int gl3_conv_heads(const void* rows, int dtype, long ld, const float*
   else if (dtype == GL3_BF16) CH_GO(bf16_t);
   else GL3_REQUIRE(false, "gl3_conv_heads: unknown dtype %d", dtype);
 #undef CH_GO
+#undef CH_TAPS
   GL3_LAUNCH_CHECK();
   return 0;
 }

@@ -486,15 +486,37 @@ extern "C" int gl3_delta_recurrence(const float* act, const float* gates, const 
 struct DeltaInner {
   int ldp, col_a, ra, col_g, rg, Rp, Na, HD, HV, D, T;
 };
-__device__ __forceinline__ void inner_store(float v, int t, int n, const DeltaInner& s, const float* __restrict__ A_log,
-                                            const float* __restrict__ dt_bias, float* __restrict__ decay, float* __restrict__ gate) {
-  if (t >= s.T) return;
-  if (n < s.Na) {
-    if (n < s.HD) decay[(long)t * s.HD + n] = expf(-expf(A_log[n / s.D]) * dr_softplus(v + dt_bias[n]));
-  } else if (n - s.Na < s.HV) {
-    gate[(long)t * s.HV + n - s.Na] = v;
+// What a lane knows of its column n of w2; `store` takes the column's sum for token t. FAST: the hardware's exponential
+// and logarithm (an error of some 1e-7 of numbers around one: 32-bit rounding of the decay itself).
+struct InnerColumn {
+  float rate, bias;
+  float* out;
+  long ld;
+  bool is_decay, exists;
+  __device__ __forceinline__ InnerColumn(int n, const DeltaInner& s, const float* A_log, const float* dt_bias, float* decay,
+                                         float* gate) {
+    is_decay = n < s.Na;
+    exists = is_decay ? n < s.HD : n - s.Na < s.HV;
+    ld = is_decay ? s.HD : s.HV;
+    out = is_decay ? decay + n : gate + (n - s.Na);
+    rate = is_decay && exists ? -expf(A_log[n / s.D]) : 0.f;
+    bias = is_decay && exists ? dt_bias[n] : 0.f;
   }
-}
+  template <bool FAST>
+  __device__ __forceinline__ void store(float v, int t, int T) const {
+    if (!exists || t >= T) return;
+    if (is_decay) {
+      v += bias;
+      if (FAST) {
+        const float sp = v > 20.f ? v : 0.6931471805599453f * __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(1.4426950408889634f * v));
+        v = __builtin_amdgcn_exp2f(1.4426950408889634f * rate * sp);
+      } else {
+        v = expf(rate * dr_softplus(v));
+      }
+    }
+    out[(long)t * ld] = v;
+  }
+};
 
 typedef __bf16 di_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float di_f32x4 __attribute__((ext_vector_type(4)));
@@ -507,13 +529,13 @@ __global__ __launch_bounds__(256) void delta_inner_mfma_kernel(const float* __re
   const int lda = s.Rp + 8;
   const int n0 = blockIdx.x * 64, t0 = blockIdx.y * 16 * MT;
   const int col = n0 < s.Na ? s.col_a : s.col_g, r = n0 < s.Na ? s.ra : s.rg;
-  for (int i = threadIdx.x; i < 16 * MT * s.Rp; i += 256) {
-    const int row = i / s.Rp, k = i % s.Rp;
-    As[row * lda + k] = static_cast<bf16_t>(k < r && t0 + row < s.T ? proj[(long)(t0 + row) * s.ldp + col + k] : 0.f);
-  }
+  for (int row = threadIdx.x >> 5; row < 16 * MT; row += 8)
+    for (int k = threadIdx.x & 31; k < s.Rp; k += 32)
+      As[row * lda + k] = static_cast<bf16_t>(k < r && t0 + row < s.T ? proj[(long)(t0 + row) * s.ldp + col + k] : 0.f);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, li = lane & 15, lq = lane >> 4;
   const int n = n0 + wave * 16 + li;
   const bf16_t* wp = w2 + (long)n * s.Rp + 8 * lq;
+  const InnerColumn mine(n, s, A_log, dt_bias, decay, gate);
   di_f32x4 acc[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) acc[m] = di_f32x4{0.f, 0.f, 0.f, 0.f};
@@ -529,7 +551,7 @@ __global__ __launch_bounds__(256) void delta_inner_mfma_kernel(const float* __re
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) inner_store(acc[m][i], t0 + 16 * m + 4 * lq + i, n, s, A_log, dt_bias, decay, gate);
+    for (int i = 0; i < 4; ++i) mine.store<true>(acc[m][i], t0 + 16 * m + 4 * lq + i, s.T);
 }
 
 __global__ __launch_bounds__(256) void delta_inner_f32_kernel(const float* __restrict__ proj, const float* __restrict__ w2,
@@ -542,7 +564,7 @@ __global__ __launch_bounds__(256) void delta_inner_f32_kernel(const float* __res
   const float* w = w2 + (long)n * s.Rp;
   float v = 0.f;
   for (int k = 0; k < r; ++k) v = fmaf(a[k], w[k], v);
-  inner_store(v, t, n, s, A_log, dt_bias, decay, gate);
+  InnerColumn(n, s, A_log, dt_bias, decay, gate).store<false>(v, t, s.T);
 }
 
 extern "C" int gl3_delta_inner(const float* proj, int ldp, int col_a, int ra, int col_g, int rg, const void* w2, int w_dtype,

@@ -74,7 +74,7 @@ extern "C" int gl3_latent_prep(const float* proj, long ld, int n_tokens, int col
               "gl3_latent_prep: null argument");
   GL3_REQUIRE(n_tokens > 0 && q_rank > 0 && rank > 0 && rot >= 0 && rot % 2 == 0 && (rot == 0 || (cos_t && sin_t)) && H > 0,
               "gl3_latent_prep: latents of %d and %d, %d rotated elements", q_rank, rank, rot);
-  GL3_REQUIRE(col_q >= 0 && col_q + q_rank <= ld && col_kv + rank + rot <= ld, "gl3_latent_prep: columns beyond the rows");
+  GL3_REQUIRE(col_q >= 0 && col_q + q_rank <= ld && (col_kv < 0 || col_kv + rank + rot <= ld), "gl3_latent_prep: columns beyond the rows");
   GL3_REQUIRE(dk >= rank + rot && dk % 16 == 0 && page_size % 32 == 0 && table_stride > 0,
               "gl3_latent_prep: cached rows of %d for %d + %d elements, pages of %d", dk, rank, rot, page_size);
   GL3_REQUIRE((long)n_tokens * H < (1L << 31), "gl3_latent_prep: too many (token, head) rows");

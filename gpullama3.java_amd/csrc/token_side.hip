@@ -21,43 +21,50 @@ __device__ __forceinline__ float side_value(float v, int t, int n, const SideGat
 }
 
 // On the matrix cores, from the 32-bit rows (rounded to bfloat16 on their way into the operand): a block takes 16 tokens x
-// 16 NT rows of W_gate, its eight waves share out K in steps of 32 and their sums are added up in wave order.
-// d must be a multiple of 8.
-template <int NT>
-__global__ __launch_bounds__(512) void side_gate_mfma_kernel(const float* __restrict__ x, const bf16_t* __restrict__ w,
-                                                             const bf16_t* __restrict__ table, const int* __restrict__ ids,
-                                                             bf16_t* __restrict__ g, SideGate s) {
-  __shared__ float part[8][NT][16][17];
+// 16 NT rows of W_gate, its NW waves share out K in runs of four steps of 32, asked for together, and their sums are added up
+// in wave order. d must be a multiple of 8. (Rows and columns that do not exist read others' numbers and are not stored.)
+template <int NT, int NW>
+__global__ __launch_bounds__(NW * 64) void side_gate_mfma_kernel(const float* __restrict__ x, const bf16_t* __restrict__ w,
+                                                                 const bf16_t* __restrict__ table, const int* __restrict__ ids,
+                                                                 bf16_t* __restrict__ g, SideGate s) {
+  __shared__ float part[NW][NT][16][17];
   const int t0 = blockIdx.x * 16, n0 = blockIdx.y * 16 * NT;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, li = lane & 15, lq = lane >> 4;
-  const bool row_ok = t0 + li < s.T;
-  const float* xp = x + (long)(row_ok ? t0 + li : 0) * s.d + 8 * lq;
+  const float* xp = x + (long)(t0 + li < s.T ? t0 + li : 0) * s.d;
   const bf16_t* wp[NT];
-  bool w_ok[NT];
   ts_f32x4 acc[NT];
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {
     const int n = n0 + 16 * nt + li;
-    w_ok[nt] = n < s.dim;
-    wp[nt] = w + (long)(w_ok[nt] ? n : 0) * s.d + 8 * lq;
+    wp[nt] = w + (long)(n < s.dim ? n : 0) * s.d;
     acc[nt] = ts_f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const ts_bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
-  for (int k = 32 * wave; k < s.d; k += 32 * 8) {
-    const bool k_ok = k + 8 * lq < s.d;
-    ts_bf16x8 a = zero;
-    if (row_ok && k_ok) {
-      const ts_f32x4 lo = *reinterpret_cast<const ts_f32x4*>(xp + k), hi = *reinterpret_cast<const ts_f32x4*>(xp + k + 4);
+  for (int k0 = 128 * wave; k0 < s.d; k0 += 128 * NW) {
+    ts_f32x4 lo[4], hi[4];
+    ts_bf16x8 b[4][NT];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        a[e] = static_cast<bf16_t>(lo[e]);
-        a[4 + e] = static_cast<bf16_t>(hi[e]);
-      }
+    for (int st = 0; st < 4; ++st) {
+      const int k = k0 + 32 * st + 8 * lq, at = k < s.d ? k : 0;
+      lo[st] = *reinterpret_cast<const ts_f32x4*>(xp + at);
+      hi[st] = *reinterpret_cast<const ts_f32x4*>(xp + at + 4);
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) b[st][nt] = *reinterpret_cast<const ts_bf16x8*>(wp[nt] + at);
     }
 #pragma unroll
-    for (int nt = 0; nt < NT; ++nt) {
-      const ts_bf16x8 b = w_ok[nt] && k_ok ? *reinterpret_cast<const ts_bf16x8*>(wp[nt] + k) : zero;
-      acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[nt], 0, 0, 0);
+    for (int st = 0; st < 4; ++st) {
+      ts_bf16x8 a;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        a[e] = static_cast<bf16_t>(lo[st][e]);
+        a[4 + e] = static_cast<bf16_t>(hi[st][e]);
+      }
+      if (k0 + 32 * st + 8 * lq >= s.d) a = zero;
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) {
+        const ts_bf16x8 bb = k0 + 32 * st + 8 * lq < s.d ? b[st][nt] : zero;
+        acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bb, acc[nt], 0, 0, 0);
+      }
     }
   }
 #pragma unroll
@@ -65,12 +72,12 @@ __global__ __launch_bounds__(512) void side_gate_mfma_kernel(const float* __rest
 #pragma unroll
     for (int i = 0; i < 4; ++i) part[wave][nt][4 * lq + i][li] = acc[nt][i];
   __syncthreads();
-  for (int i = threadIdx.x; i < NT * 256; i += 512) {
+  for (int i = threadIdx.x; i < NT * 256; i += NW * 64) {
     const int r = i / (16 * NT), c = i % (16 * NT), n = n0 + c, t = t0 + r;
     if (t >= s.T || n >= s.dim_pad) continue;
     float v = 0.f;
 #pragma unroll
-    for (int wv = 0; wv < 8; ++wv) v += part[wv][c >> 4][r][c & 15];
+    for (int wv = 0; wv < NW; ++wv) v += part[wv][c >> 4][r][c & 15];
     g[(long)t * s.ldg + n] = static_cast<bf16_t>(side_value<bf16_t>(v, t, n, s, ids, table));
   }
 }
@@ -98,11 +105,11 @@ extern "C" int gl3_side_gate(const float* x, const void* w, int dtype, const voi
   if (dtype == GL3_BF16 && mfma && d % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0) {
     const unsigned tiles = (unsigned)((T + 15) / 16);
     if (T <= 256)
-      side_gate_mfma_kernel<1><<<dim3(tiles, (dim_pad + 15) / 16), dim3(512), 0, stream>>>(x, (const bf16_t*)w, (const bf16_t*)table, ids,
-                                                                                          (bf16_t*)g, s);
+      side_gate_mfma_kernel<1, 16><<<dim3(tiles, (dim_pad + 15) / 16), dim3(1024), 0, stream>>>(x, (const bf16_t*)w, (const bf16_t*)table,
+                                                                                               ids, (bf16_t*)g, s);
     else
-      side_gate_mfma_kernel<2><<<dim3(tiles, (dim_pad + 31) / 32), dim3(512), 0, stream>>>(x, (const bf16_t*)w, (const bf16_t*)table, ids,
-                                                                                          (bf16_t*)g, s);
+      side_gate_mfma_kernel<2, 8><<<dim3(tiles, (dim_pad + 31) / 32), dim3(512), 0, stream>>>(x, (const bf16_t*)w, (const bf16_t*)table,
+                                                                                             ids, (bf16_t*)g, s);
   } else {
     const dim3 grid(T, (dim_pad + 3) / 4), block(256);
     if (dtype == GL3_F32) side_gate_kernel<float><<<grid, block, 0, stream>>>(x, (const float*)w, (const float*)table, ids, (float*)g, s);

@@ -191,20 +191,25 @@ def expert(h, W, p, limit, r=exact):
     return linear(r(g * sigmoid(1.702 * g) * (u + 1.0)), W[p + "down"])
 
 
-def choose(c, router):
-    """The chosen experts of ONE token from its choice scores c [experts], and how far the nearest other choice lies
-    (the scores' margin of the last group kept and of the last expert chosen)."""
+def choose(c, router, s=None):
+    """The chosen experts of ONE token from its choice scores c [experts], and the margin of the choice: by how much the
+    last group kept and the last expert chosen lie above the next ones, with ``s`` (the scores themselves) as a fraction of
+    the larger score of the two that compete, which is what a rounding moves."""
     E, top, groups = router["experts"], router["top"], router.get("groups") or {"count": 1, "keep": 1}
     n, keep = groups["count"], groups["keep"]
-    best = c.reshape(n, E // n).max(-1)
-    order = np.argsort(-best, kind="stable")
+
+    def margin(a, b):
+        return (c[a] - c[b]) / (1.0 if s is None else max(s[a], s[b]))
+
+    leaders = c.reshape(n, E // n).argmax(-1) + np.arange(n) * (E // n)
+    order = np.argsort(-c[leaders], kind="stable")
     open_ = np.zeros(n, bool)
     open_[order[:keep]] = True
     left = np.where(np.repeat(open_, E // n), c, -np.inf)
     ranked = np.argsort(-left, kind="stable")
-    gap = best[order[keep - 1]] - best[order[keep]] if keep < n else math.inf
-    if top < E:
-        gap = min(gap, left[ranked[top - 1]] - left[ranked[top]])
+    gap = margin(leaders[order[keep - 1]], leaders[order[keep]]) if keep < n else math.inf
+    if top < E and left[ranked[top]] > -np.inf:
+        gap = min(gap, margin(ranked[top - 1], ranked[top]))
     return ranked[:top], gap
 
 
@@ -215,7 +220,7 @@ def route(h, W, p, router):
     s = s / s.sum(-1, keepdims=True)
     out = []
     for row in s:
-        idx, gap = choose(row + W[p + "correction"], router)
+        idx, gap = choose(row + W[p + "correction"], router, row)
         out.append((idx, row[idx] / (row[idx].sum() + 1e-20) * router["scale"], gap))
     return out
 
@@ -376,7 +381,7 @@ def make_weights(cfg, seed, ranks=lambda i: (8, 12), overrides=None):
     return out
 
 
-def tokens_with_clear_choices(cfg, W, seed, n, gap=0.01):
+def tokens_with_clear_choices(cfg, W, seed, n, gap=0.12):
     """n token ids drawn from a seed at which no router makes a close call: at every token and layer the margin of the
     groups and of the experts (``choose``) is at least ``gap``, so an engine that rounds to 16 bits chooses the same
     experts."""
@@ -393,7 +398,7 @@ def tokens_with_clear_choices(cfg, W, seed, n, gap=0.01):
                 best = (least, t, trial)
             if least >= gap:
                 break
-        if best[0] < gap / 5:
+        if best[0] < gap / 4:
             raise RuntimeError("no token without a close call found")
         seq = best[2]
         out.append(best[1])
