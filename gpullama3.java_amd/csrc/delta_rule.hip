@@ -105,32 +105,34 @@ __global__ __launch_bounds__(256) void delta_conv_state_kernel(const float* __re
   }
 }
 
-// The rule itself and the read-out's norm. grid (H, B, blocks a head: 1 unless the launcher deals a prompt's head out), a block of ceil(Dv / 16) waves: wave w owns the 16 value
-// columns 16 w .. of head h's matrix, lane (r, c) of it the rows r, r + 4, ... of column c (RPL rows a lane), so a
-// token costs a lane RPL multiply-adds for each of S^T k, the update and S^T q, and the sums over the four lanes of
-// a column are two lane swaps each (no trip through shared memory). The tokens' operands (k, q, v, decay,
-// strength) come in chunks of DR_CHUNK tokens through shared memory, the next chunk's loads on their way while
-// the current chunk is worked on: what a token waits for is its own chain of multiply-adds, not memory.
-// After the last token the block divides each of its tokens' read-outs (which it wrote to `o` itself) by their
-// root mean square over the head and applies the weight and the gate: y = o / rms * w * silu(gate).
+// The rule itself and the read-out's norm. grid (H, B, blocks a head: more than one where the launcher deals a prompt's head
+// out), a wave owns 64 / RG value columns of head h's matrix, lane (r, c) of it the rows r, r + RG, ... of column c (RPL rows a
+// lane), so a token costs a lane RPL multiply-adds for each of S^T k, the update and S^T q, and the sums over the lanes of
+// a column are lane moves (no trip through shared memory). The tokens' operands (k, q, v, decays, strength) come in chunks
+// of DR_CHUNK tokens through shared memory, the next chunk's loads on their way while the current chunk is worked on: what a
+// token waits for is a wave's own instructions, not memory.
+// Steps of few tokens: after the last token the block divides each of its tokens' read-outs (which it wrote to `o` itself) by
+// their root mean square over the head and applies the weight and the gate: y = o / rms * w * silu(gate).
 #define DR_CHUNK 16   // the most tokens a chunk; the launcher takes fewer where keys and values are long
 #define DR_NLD 8       // loads a thread has on their way for the next chunk (with decays per channel DR_NLD_CH)
 #define DR_NLD_CH 10
 
-__device__ __forceinline__ float dr_sum4(float p) {   // the sum over lanes l, l ^ 16, l ^ 32, l ^ 48
-  auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(p), __float_as_uint(p), false, false);
-  p = __uint_as_float(a[0]) + __uint_as_float(a[1]);
-  auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(p), __float_as_uint(p), false, false);
-  return __uint_as_float(b[0]) + __uint_as_float(b[1]);
-}
-
-// RG: the lanes a column's rows are dealt out to, 4 (16 columns a wave) or 8 (8 columns a wave: twice the waves with
-// half the work per token each, which is what a prompt's long chains of tokens want; the state lies the same).
+// Two sums at once over the RG lanes that share a column (lanes 64 / RG apart): both values travel together, p in the lower
+// half of the wave and o in the upper, until both sums are in every lane. RG: the lanes a column's rows are dealt out to, 4, 8
+// or 16 (16, 8 or 4 columns a wave; the state lies the same).
 template <int RG>
-__device__ __forceinline__ float dr_sum_rows(float p) {
-  if (RG == 8)    // lane l ^ 8 is 8 places round the row of 16
-    p += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(p), 0x128, 0xf, 0xf, false));
-  return dr_sum4(p);
+__device__ __forceinline__ void dr_sum_pair(float& p, float& o) {
+  auto a = __builtin_amdgcn_permlane32_swap(__float_as_uint(p), __float_as_uint(o), false, false);
+  float x = __uint_as_float(a[0]) + __uint_as_float(a[1]);      // p over lanes l, l + 32; o the same in the upper half
+  if (RG >= 8)    // lane l ^ 8 is 8 places round the row of 16
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));
+  if (RG == 16)   // then lanes 8 apart hold the same: 4 places round the row are the other two
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x124, 0xf, 0xf, false));
+  a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  x = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  a = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  p = __uint_as_float(a[0]);
+  o = __uint_as_float(a[1]);
 }
 
 __device__ __forceinline__ float dr_gate(float z, int sigmoid) { return sigmoid ? dr_sigmoid(z) : z * dr_sigmoid(z); }
@@ -143,7 +145,7 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
     const float* __restrict__ proj, int ldp, int off_gate, const float* __restrict__ norm_w, TO* __restrict__ y,
     float eps, DeltaShape s, int chunk, int norm_here, int own_waves, int gate_sigmoid) {
   constexpr int NLD = CH ? DR_NLD_CH : DR_NLD;
-  extern __shared__ __attribute__((aligned(16))) float dr_lds[];   // two buffers of chunk * per_token floats
+  extern __shared__ __attribute__((aligned(16))) float dr_lds[];   // two buffers of chunk * per_token floats, and one token more
   typedef float f4 __attribute__((ext_vector_type(4)));
   const int h = blockIdx.x, b = blockIdx.y;
   constexpr int COLS = 64 / RG;
@@ -175,111 +177,136 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
   const int n_src = chunk * per_src;
   const long q_at = (long)kvh * D, k_at = (long)s.G * D + (long)kvh * D, v_at = 2L * s.G * D + (long)h * Dv;
   const int threads = blockDim.x;
-  for (int e = tid; e < 2 * chunk * per_token; e += threads) dr_lds[e] = 0.f;
+  for (int e = tid; e < (2 * chunk + 1) * per_token; e += threads) dr_lds[e] = 0.f;      // (one token more: see the reads ahead)
   __syncthreads();
-  float held[NLD];
-  auto ask = [&](int t0) {
+  // This thread's places: place n of a chunk is operand e = tid + n threads of the chunk's per_src a token. Where it comes
+  // from in the first chunk, how far that moves on from chunk to chunk, and where it goes are worked out once.
+  float held[NLD] = {};
+  const float* from[NLD];
+  int step[NLD], to[NLD];
+#pragma unroll
+  for (int n = 0; n < NLD; ++n) {
+    const int e = tid + n * threads;
+    const int tt = e / per_src, f = e - tt * per_src;
+    const long t = first + tt;
+    int at;
+    if (f < NV * D) {
+      const int which = CH && f >= 2 * D ? 2 : f >= D, i = f - which * D;
+      at = which * VEC + (i % RG) * RPL + i / RG;
+      from[n] = which == 2 ? decay + t * H * D + (long)h * D + i : act + t * C + (which ? k_at : q_at) + i;
+      step[n] = (which == 2 ? H * D : C) * chunk;
+    } else {
+      at = NV * VEC + (f - NV * D);
+      const bool value = f < NV * D + Dv;
+      from[n] = value ? act + t * C + v_at + (f - NV * D) : gates + t * 2 * H + (long)(CH ? 1 : f - 2 * D - Dv) * H + h;
+      step[n] = (value ? C : 2 * H) * chunk;
+    }
+    to[n] = tt * per_token + at;
+  }
+  auto ask = [&](int t0) {      // (called for one chunk after the other)
+    const int here = min(n_src, (last - t0) * per_src);
 #pragma unroll
     for (int n = 0; n < NLD; ++n) {
-      const int e = tid + n * threads;
-      const int tt = e / per_src, f = e - tt * per_src, t = t0 + tt;
-      const float* p = act;
-      if (e < n_src && t < last) {
-        if (f < D) p = act + (long)t * C + q_at + f;
-        else if (f < 2 * D) p = act + (long)t * C + k_at + (f - D);
-        else if (CH && f < 3 * D) p = decay + (long)t * H * D + (long)h * D + (f - 2 * D);
-        else if (f < NV * D + Dv) p = act + (long)t * C + v_at + (f - NV * D);
-        else p = gates + (long)t * 2 * H + (long)(CH ? 1 : f - 2 * D - Dv) * H + h;
-      }
-      held[n] = *p;
+      if (tid + n * threads < here) held[n] = *from[n];
+      from[n] += step[n];
     }
   };
   auto put = [&](int buf) {
 #pragma unroll
-    for (int n = 0; n < NLD; ++n) {
-      const int e = tid + n * threads;
-      if (e < n_src) {
-        const int tt = e / per_src, f = e - tt * per_src;
-        int at;
-        if (f < NV * D) {
-          const int which = CH && f >= 2 * D ? 2 : f >= D, i = f - which * D;
-          at = which * VEC + (i % RG) * RPL + i / RG;
-        } else {
-          at = NV * VEC + (f - NV * D);
-        }
-        dr_lds[(buf * chunk + tt) * per_token + at] = held[n];
-      }
-    }
+    for (int n = 0; n < NLD; ++n)
+      if (tid + n * threads < n_src) dr_lds[buf * chunk * per_token + to[n]] = held[n];
   };
   ask(first);
   put(0);
   __syncthreads();
-  int buf = 0;
+  // A token's read-out is made in the pass of the token after it, with the matrix as it stands then: its sum over the rows
+  // and the next token's S^T k are one reduction. So a pass takes k, decay, v and strength of its own token and q of the one
+  // before (zeros for the first: the buffers were cleared), and stores the read-out of the one before.
+  struct Operands { float k[RPL], q[RPL], gs[CH ? RPL : 1], v, beta; };
+  const int lane_at = r * RPL, v_place = NV * VEC + (valid ? j : 0);
+  auto fetch = [&](Operands& x, int at, int q_from) {      // (places of the token's operands, and of the token's before it)
+    const float *op = dr_lds + at, *oq = dr_lds + q_from + lane_at;
+#pragma unroll
+    for (int ii = 0; ii < RPL; ii += 4) {
+      const f4 q4 = *(const f4*)(oq + ii), k4 = *(const f4*)(op + lane_at + VEC + ii);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) { x.q[ii + e] = q4[e]; x.k[ii + e] = k4[e]; }
+      if constexpr (CH) {
+        const f4 g4 = *(const f4*)(op + lane_at + 2 * VEC + ii);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x.gs[ii + e] = g4[e];
+      }
+    }
+    if constexpr (!CH) x.gs[0] = op[NV * VEC + Dv];
+    x.beta = op[NV * VEC + Dv + (CH ? 0 : 1)];
+    x.v = op[v_place];
+  };
+  float* read_out = o + (long)first * H * Dv + (long)h * Dv + j;
+  int advance = 0;                       // (the first pass has no read-out to store: its zero lands where the second's goes)
+  const bool whole = __all(valid);
+  auto store = [&](float v) {            // (all lanes of a column hold the same number)
+    if (whole) *read_out = v;
+    else if (valid) *read_out = v;
+    read_out += advance;
+    advance = H * Dv;
+  };
+  auto work = [&](const Operands& x) {
+    float p2[2] = {0.f, 0.f}, o2[2] = {0.f, 0.f};
+#pragma unroll
+    for (int ii = 0; ii < RPL; ++ii) {
+      o2[ii & 1] = fmaf(S[ii], x.q[ii], o2[ii & 1]);
+      S[ii] *= x.gs[CH ? ii : 0];
+      p2[ii & 1] = fmaf(S[ii], x.k[ii], p2[ii & 1]);
+    }
+    float part = p2[0] + p2[1], read = o2[0] + o2[1];
+    dr_sum_pair<RG>(part, read);
+    const float uu = valid ? x.beta * (x.v - part) : 0.f;
+#pragma unroll
+    for (int ii = 0; ii < RPL; ++ii) S[ii] = fmaf(x.k[ii], uu, S[ii]);
+    store(read);
+  };
+  int buf = 0, q_last = (2 * chunk - 1) * per_token;
   for (int t0 = first; t0 < last; t0 += chunk) {
     const bool more = t0 + chunk < last;
     if (more) ask(t0 + chunk);
     const int n_here = min(chunk, last - t0);
-    // two tokens' operands in registers in turn: the next token's reads from shared memory are on their way while
-    // the current token's chain of multiply-adds runs
-    struct Operands { float k[RPL], q[RPL], gs[CH ? RPL : 1], v, beta; };
-    auto fetch = [&](Operands& x, int tt) {
-      const float* op = dr_lds + (buf * chunk + tt) * per_token;
-#pragma unroll
-      for (int ii = 0; ii < RPL; ii += 4) {
-        const f4 q4 = *(const f4*)(op + r * RPL + ii), k4 = *(const f4*)(op + VEC + r * RPL + ii);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) { x.q[ii + e] = q4[e]; x.k[ii + e] = k4[e]; }
-        if constexpr (CH) {
-          const f4 g4 = *(const f4*)(op + 2 * VEC + r * RPL + ii);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) x.gs[ii + e] = g4[e];
-        }
-      }
-      if constexpr (!CH) x.gs[0] = op[NV * VEC + Dv];
-      x.beta = op[NV * VEC + Dv + (CH ? 0 : 1)];
-      x.v = valid ? op[NV * VEC + j] : 0.f;
-    };
-    auto work = [&](const Operands& x, int tt) {
-      float p4[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ii = 0; ii < RPL; ++ii) {
-        S[ii] *= x.gs[CH ? ii : 0];
-        p4[ii & 3] = fmaf(S[ii], x.k[ii], p4[ii & 3]);
-      }
-      const float part = dr_sum_rows<RG>((p4[0] + p4[1]) + (p4[2] + p4[3]));
-      const float uu = x.beta * (x.v - part);
-      float o4[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ii = 0; ii < RPL; ++ii) {
-        S[ii] = fmaf(x.k[ii], uu, S[ii]);
-        o4[ii & 3] = fmaf(S[ii], x.q[ii], o4[ii & 3]);
-      }
-      const float read = dr_sum_rows<RG>((o4[0] + o4[1]) + (o4[2] + o4[3]));
-      if (r == 0 && valid) o[(long)(t0 + tt) * H * Dv + (long)h * Dv + j] = read;
-    };
+    int at = buf * chunk * per_token;
+    Operands xa;
+    fetch(xa, at, q_last);
     if constexpr (RPL <= (CH ? 16 : 24) && MAXT <= 512) {
-      // (pairs of tokens without a branch between them, so that the end of one token's work, which nothing waits
-      // for, can be scheduled into the start of the next one's)
-      Operands xa, xb;
-      fetch(xa, 0);
+      // (two tokens' operands in registers in turn: the next token's reads from shared memory are on their way while the
+      // current token's chain of multiply-adds runs; the read behind a chunk's last token is of no use and does no harm)
+      Operands xb;
       int tt = 0;
       for (; tt + 2 <= n_here; tt += 2) {
-        fetch(xb, tt + 1);
-        work(xa, tt);
-        fetch(xa, min(tt + 2, n_here - 1));
-        work(xb, tt + 1);
+        fetch(xb, at + per_token, at);
+        work(xa);
+        fetch(xa, at + 2 * per_token, at + per_token);
+        work(xb);
+        at += 2 * per_token;
       }
-      if (tt < n_here) work(xa, tt);
+      if (tt < n_here) {
+        work(xa);
+        at += per_token;
+      }
     } else {                              // (long keys, or a block of sixteen waves: two tokens' operands beside the matrix do not fit the registers)
-      Operands xa;
       for (int tt = 0; tt < n_here; ++tt) {
-        fetch(xa, tt);
-        work(xa, tt);
+        if (tt > 0) fetch(xa, at, at - per_token);
+        work(xa);
+        at += per_token;
       }
     }
+    q_last = at - per_token;              // (the next chunk is put beside this one, not over it)
     if (more) put(buf ^ 1);
     __syncthreads();
     buf ^= 1;
+  }
+  {                                       // the last token's read-out
+    float read = 0.f, none = 0.f;
+#pragma unroll
+    for (int ii = 0; ii < RPL; ++ii) read = fmaf(S[ii], dr_lds[q_last + lane_at + ii], read);
+    dr_sum_pair<RG>(none, read);
+    store(read);
   }
 #pragma unroll
   for (int ii = 0; ii < RPL; ++ii) {
@@ -307,6 +334,85 @@ __global__ __launch_bounds__(MAXT) void delta_recurrence_kernel(
       const float z = grow[e];
       dst[e] = from_f32<TO>(orow[e] * f * norm_w[e] * dr_gate(z, gate_sigmoid));
     }
+  }
+}
+
+// The same for a step in which every sequence brings ONE token: the time is the matrices' way from memory and back. A block
+// a (head, sequence), a wave a tile of 16 columns; lane (r, c) holds 4 consecutive columns 4 c of the rows r, r + 16, ... (16
+// bytes each, a wave 1 KB of consecutive memory), and reads its rows' operands straight from memory. At the end the block
+// norms the head's read-outs, which stay in shared memory. IT: 16ths of the rows, rounded up.
+template <int IT, typename TO, bool CH>
+__global__ __launch_bounds__(1024) void delta_one_token_kernel(
+    const float* __restrict__ act, const float* __restrict__ gates, const float* __restrict__ decay, float* __restrict__ state,
+    const int* __restrict__ slot_ids, const float* __restrict__ proj, int ldp, int off_gate, const float* __restrict__ norm_w,
+    TO* __restrict__ y, float eps, DeltaShape s, int gate_sigmoid) {
+  typedef float f4 __attribute__((ext_vector_type(4)));
+  __shared__ float read[256];
+  __shared__ float scratch[16];
+  const int h = blockIdx.x, t = blockIdx.y, tile = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane >> 2, c = (lane & 3) * 4;
+  const int D = s.D, H = s.H, Dv = s.Dv, C = 2 * s.G * D + H * Dv, CT = (Dv + 15) / 16;
+  float* mat = state + (long)slot_ids[t] * s.state_stride + ((long)(h * CT + tile) * D) * 16 + c;
+  const float* row = act + (long)t * C;
+  const float* qp = row + (long)(h / (H / s.G)) * D;
+  const float* kp = qp + (long)s.G * D;
+  f4 S[IT];
+  float k[IT], q[IT], g[CH ? IT : 1];
+#pragma unroll
+  for (int n = 0; n < IT; ++n) {
+    const int i = r + 16 * n;
+    const bool ok = i < D;
+    S[n] = ok ? *(const f4*)(mat + (long)i * 16) : f4{0.f, 0.f, 0.f, 0.f};
+    k[n] = ok ? kp[i] : 0.f;
+    q[n] = ok ? qp[i] : 0.f;
+    if (CH) g[n] = ok ? decay[(long)t * H * D + (long)h * D + i] : 0.f;
+  }
+  if (!CH) g[0] = gates[(long)t * 2 * H + h];
+  const float beta = gates[(long)t * 2 * H + H + h];
+  float v[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = tile * 16 + c + e < Dv ? row[2L * s.G * D + (long)h * Dv + tile * 16 + c + e] : 0.f;
+  auto over_rows = [](f4 p) {            // the sum over the 16 lanes that hold the same columns
+#pragma unroll
+    for (int o = 4; o < 64; o <<= 1)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) p[e] += __shfl_xor(p[e], o, 64);
+    return p;
+  };
+  f4 p = {0.f, 0.f, 0.f, 0.f}, out = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int n = 0; n < IT; ++n) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      S[n][e] *= g[CH ? n : 0];
+      p[e] = fmaf(S[n][e], k[n], p[e]);
+    }
+  }
+  p = over_rows(p);
+  float u[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) u[e] = beta * (v[e] - p[e]);
+#pragma unroll
+  for (int n = 0; n < IT; ++n) {
+    const int i = r + 16 * n;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      S[n][e] = fmaf(k[n], u[e], S[n][e]);
+      out[e] = fmaf(S[n][e], q[n], out[e]);
+    }
+    if (i < D) *(f4*)(mat + (long)i * 16) = S[n];
+  }
+  out = over_rows(out);
+  if (r == 0) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) read[tile * 16 + c + e] = out[e];
+  }
+  __syncthreads();
+  const int j = threadIdx.x;
+  const float o = j < Dv ? read[j] : 0.f;
+  const float f = 1.0f / sqrtf(block_sum(o * o, scratch) / (float)Dv + eps);
+  if (j < Dv) {
+    const float z = proj[(long)t * ldp + off_gate + (long)h * Dv + j];
+    y[((long)t * H + h) * Dv + j] = from_f32<TO>(o * f * norm_w[j] * dr_gate(z, gate_sigmoid));
   }
 }
 
@@ -378,11 +484,12 @@ extern "C" int gl3_delta_prep(const float* proj, const float* conv_w, const floa
 // act [T][C], gates [T][2 H] as gl3_delta_prep left them. o [T][H Dv] float receives the raw read-outs (scratch);
 // y [T][H Dv] (float or bfloat16) the read-outs divided by their root mean square over each head, times norm_w [Dv]
 // (float), times silu of the gate (gate_sigmoid: sigmoid), whose H Dv columns start at off_gate of proj [T][ldp] (float).
-// decay [T][H D] (may be null): a factor per key channel, in place of the heads' decays in gates.
+// decay [T][H D] (may be null): a factor per key channel, in place of the heads' decays in gates. one_each: every sequence
+// brings exactly one token (o is then left alone where the slots' states lie at multiples of 16 bytes).
 extern "C" int gl3_delta_recurrence(const float* act, const float* gates, const float* decay, float* state, const int* cu_seqlens,
                                     const int* slot_ids, float* o, const float* proj, int ldp, int off_gate,
                                     const float* norm_w, void* y, int y_dtype, float eps, int T, int B, int H, int G, int D,
-                                    int Dv, int taps, long state_stride, int gate_sigmoid, hipStream_t stream) {
+                                    int Dv, int taps, long state_stride, int gate_sigmoid, int one_each, hipStream_t stream) {
   if (B == 0 || T == 0) return 0;
   GL3_REQUIRE(act && gates && state && cu_seqlens && slot_ids && o && proj && norm_w && y && B > 0,
               "gl3_delta_recurrence: bad arguments");
@@ -392,34 +499,62 @@ extern "C" int gl3_delta_recurrence(const float* act, const float* gates, const 
   GL3_REQUIRE(Dv <= 256, "gl3_delta_recurrence: values of %d elements: a block holds up to 256 columns", Dv);
   GL3_REQUIRE(off_gate >= 0 && off_gate + H * Dv <= ldp, "gl3_delta_recurrence: the gate's columns %d .. of rows of %d", off_gate, ldp);
   GL3_REQUIRE(y_dtype == GL3_F32 || y_dtype == GL3_BF16, "gl3_delta_recurrence: unknown dtype %d", y_dtype);
+  GL3_REQUIRE(!one_each || T == B, "gl3_delta_recurrence: %d tokens of %d sequences are not one each", T, B);
+  if (one_each && state_stride % 4 == 0 && (uintptr_t)state % 16 == 0) {
+    const dim3 grid1(H, B), block1((Dv + 15) / 16 * 64);
+#define ONE3(IT, TO, CH)                                                                                                    \
+  delta_one_token_kernel<IT, TO, CH><<<grid1, block1, 0, stream>>>(act, gates, decay, state, slot_ids, proj, ldp, off_gate, \
+                                                                   norm_w, (TO*)y, eps, s, gate_sigmoid)
+#define ONE2(IT, TO)                     \
+  do {                                   \
+    if (decay) ONE3(IT, TO, true);       \
+    else ONE3(IT, TO, false);            \
+  } while (0)
+#define ONE(IT)                                  \
+  do {                                           \
+    if (y_dtype == GL3_F32) ONE2(IT, float);     \
+    else ONE2(IT, bf16_t);                       \
+  } while (0)
+    if (D <= 32) ONE(2);
+    else if (D <= 64) ONE(4);
+    else if (D <= 128) ONE(8);
+    else ONE(16);
+#undef ONE
+#undef ONE2
+#undef ONE3
+    GL3_LAUNCH_CHECK();
+    return 0;
+  }
   // as many waves as the columns need, and as the loads of a chunk of operands need (DR_NLD a thread)
   // the read-outs' norm: by the block that made them where a sequence brings few tokens (a decode step), else by a
   // launch of its own with a wave to every token and head (a block's few waves would walk a prompt's tokens one by one)
   const int norm_here = T <= 4 * B;
-  // a column's rows over 8 lanes for prompts (long chains of tokens: half the work per token and wave) where that
-  // makes at most eight waves, over 4 else (values of 128: sixteen waves of 8 columns were 5% slower than eight of 16)
-  const int rg = (!norm_here && D >= 32 && Dv <= 64) ? 8 : 4;
+  // A prompt's chain of tokens is bound by a wave's instructions per token: the fewer rows a lane, the fewer of them (one
+  // prompt of 2,048 tokens, 32 heads of 64 and decays per channel: 4 lanes a column 690 us, 8 lanes 500, 16 lanes 400), in blocks
+  // of at most eight waves, a head's columns dealt out to several blocks (grid z) if need be. Where sequences enough run
+  // side by side to fill the chip, 8 lanes: their total of instructions is less (eight sequences of 512 tokens: 176 against 200).
+  // Steps of few tokens a sequence: 4 lanes, a block a head, which norms the head's read-outs itself.
+  auto blocks_a_head = [&](int lanes) { return ((long)Dv * lanes + 64 * 8 - 1) / (64 * 8); };
+  const int rg = norm_here || D < 32 ? 4 : D >= 48 && (long)H * B * blocks_a_head(16) <= 256 ? 16 : 8;
   const int cols = 64 / rg;
-  // (fewer tokens a chunk where that keeps the block at the waves its columns need, or at four)
-  // (A head's columns could be dealt out to several blocks, grid z; with blocks of four waves of 8 columns a prompt of
-  // 2,048 tokens was slower than with one block of eight, 12.8 against 12.1 ms for sixteen layers: every block stages
-  // all of a token's operands, in shorter chunks. One block a head.)
   const int all_col_waves = (Dv + cols - 1) / cols;
-  const int col_waves = all_col_waves;
-  const int split = 1;
+  const int want = norm_here ? 1 : (int)blocks_a_head(rg);
+  const int col_waves = (all_col_waves + want - 1) / want;
+  const int split = (all_col_waves + col_waves - 1) / col_waves;
+  // (fewer tokens a chunk where that keeps the block at the waves its columns need, or at four)
   const int nv = decay ? 3 : 2, nld = decay ? DR_NLD_CH : DR_NLD, per_src = nv * D + Dv + (decay ? 1 : 2);
   int chunk = DR_CHUNK, waves = col_waves;
   const int rows = (D + rg - 1) / rg;
   const int rpl = rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : rows <= 24 ? 24 : rows <= 32 ? 32 : rows <= 48 ? 48 : 64;
-  const size_t lds_token = 2 * (size_t)(nv * rg * rpl + ((Dv + 2 + 3) & ~3)) * sizeof(float);
+  const size_t lds_token = (size_t)(nv * rg * rpl + ((Dv + 2 + 3) & ~3)) * sizeof(float);
   for (;; chunk /= 2) {
     waves = col_waves;
     while (waves * 64 * nld < chunk * per_src) ++waves;
-    if ((waves <= (col_waves > 4 ? col_waves : 4) && chunk * lds_token <= 64 * 1024) || chunk == 1) break;
+    if ((waves <= (col_waves > 4 ? col_waves : 4) && (2 * chunk + 1) * lds_token <= 64 * 1024) || chunk == 1) break;
   }
   GL3_REQUIRE(waves <= 16, "gl3_delta_recurrence: keys of %d with values of %d need more than a block's threads", D, Dv);
   dim3 grid(H, B, split), block(waves * 64);
-  const size_t lds = chunk * lds_token;
+  const size_t lds = (2 * chunk + 1) * lds_token;
   GL3_REQUIRE(lds <= 64 * 1024, "gl3_delta_recurrence: a chunk's operands of %zu bytes exceed shared memory", lds);
 #define GO5(R, TO, MAXT, RGV, CH)                                                                                          \
   delta_recurrence_kernel<R, TO, MAXT, RGV, CH><<<grid, block, lds, stream>>>(                                             \
@@ -432,6 +567,9 @@ extern "C" int gl3_delta_recurrence(const float* act, const float* gates, const 
   } while (0)
 #define GO3(R, TO, MAXT)                                                       \
   do {                                                                         \
+    if constexpr (R <= 16) {                                                   \
+      if (rg == 16) { GO4(R, TO, MAXT, 16); break; }                           \
+    }                                                                          \
     if constexpr (R <= 32) {                                                   \
       if (rg == 8) { GO4(R, TO, MAXT, 8); break; }                             \
     }                                                                          \

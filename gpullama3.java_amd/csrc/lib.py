@@ -90,7 +90,7 @@ def _declare(lib):
         "gl3_residual_inject": [P, P, P, I, I, P],
         "gl3_delta_state_floats": [I, I, I, I, I],
         "gl3_delta_prep": [P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, I, I, L, F, F, I, P],
-        "gl3_delta_recurrence": [P, P, P, P, P, P, P, P, I, I, P, P, I, F, I, I, I, I, I, I, I, L, I, P],
+        "gl3_delta_recurrence": [P, P, P, P, P, P, P, P, I, I, P, P, I, F, I, I, I, I, I, I, I, L, I, I, P],
         "gl3_delta_inner": [P, I, I, I, I, I, P, I, I, I, I, P, P, P, P, I, I, I, I, P],
         "gl3_conv_heads": [P, I, L, P, I, P, L, L, P, P, P, P, P, P, I, P, P, I, P, P, I, F, P, P, P, I, I, I, I, I, I, I, I, P],
         "gl3_side_gate": [P, P, I, P, L, I, P, P, L, I, I, I, I, I, I, P],
@@ -1273,11 +1273,12 @@ def delta_prep(proj, offsets, conv_w, A_log, dt_bias, state, cu_seqlens, seq_of_
 
 
 def delta_recurrence(act, gates, state, cu_seqlens, slot_ids, readout, proj, off_gate, norm_w, out, H, G, D, Dv, taps, eps,
-                     decay=None, gate_act="silu"):
+                     decay=None, gate_act="silu", one_token_each=False):
     """The rule itself, token by token for every sequence of the step from the state it holds, then the read-outs'
     norm: ``out[t, h] = o[t, h] / rms * norm_w * silu(gate[t, h])`` (``out`` [T, H Dv] float32 or bfloat16), the gate in
     columns ``off_gate`` .. of ``proj``; ``readout`` [T, H Dv] float32 is scratch for the raw read-outs. ``decay`` [T, H D]
-    float32: a factor per key channel in place of the heads' decays; ``gate_act``: "silu" or "sigmoid"."""
+    float32: a factor per key channel in place of the heads' decays; ``gate_act``: "silu" or "sigmoid". ``one_token_each``: the
+    caller vouches that every sequence brings exactly one token (a kernel of its own; ``readout`` may then stay as it is)."""
     _dev(act, "act", torch.float32); _dev(gates, "gates", torch.float32); _dev(readout, "readout", torch.float32)
     _dev(proj, "proj", torch.float32, contiguous=False); _dev(norm_w, "norm_w", torch.float32); _dev(out, "out")
     T = act.shape[0]
@@ -1296,7 +1297,8 @@ def delta_recurrence(act, gates, state, cu_seqlens, slot_ids, readout, proj, off
     _check(library().gl3_delta_recurrence(_ptr(act), _ptr(gates), _ptr(decay), _ptr(state), _ptr(cu_seqlens), _ptr(slot_ids),
                                           _ptr(readout), _ptr(proj), proj.stride(0), off_gate, _ptr(norm_w), _ptr(out),
                                           _code(out, "out"), float(eps), T, B, H, G, D, Dv, taps, state.stride(0),
-                                          int(gate_act == "sigmoid"), _stream()), "delta_recurrence")
+                                          int(gate_act == "sigmoid"), int(bool(one_token_each) and T == B), _stream()),
+           "delta_recurrence")
 
 
 def delta_inner(proj, col_a, rank_a, col_g, rank_g, w2, rows_a, A_log, dt_bias, decay, gate, H, D, Dv):

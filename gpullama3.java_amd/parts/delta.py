@@ -115,7 +115,7 @@ class GatedDeltaRule:
         return None
 
     def state_need(self):
-        return StateNeed(K.delta_state_floats(self.H, self.G, self.D, self.Dv, self.taps), torch.float32)
+        return StateNeed(-(-K.delta_state_floats(self.H, self.G, self.D, self.Dv, self.taps) // 4) * 4, torch.float32)
 
     def forward(self, ctx, h, x, run, epilogue=ops.EPI_ADD):
         """``epilogue``: EPI_ADD adds the output into the residual rows ``x``; EPI_STORE writes it to ``x``, a float32
@@ -126,6 +126,7 @@ class GatedDeltaRule:
         ops.linear(h, self.w_in, proj, ops.EPI_STORE, ctx)
         act = ctx.buffer("delta_act", (T, self.channels), torch.float32)
         gates = ctx.buffer("delta_gates", (T, 2 * H), torch.float32)
+        one_each = bool(ctx.decode and ctx.max_q_len == 1)
         decay, gate, off_gate = None, proj, self.off_g
         if self.two_step:
             decay = ctx.buffer("delta_decay", (T, H * D), torch.float32)
@@ -135,11 +136,11 @@ class GatedDeltaRule:
         K.delta_prep(proj, (self.off_q, self.off_k, self.off_v, self.off_b, self.off_a), self.conv_w,
                      None if self.two_step else self.A_log, None if self.two_step else self.dt_bias,
                      state, ctx.cu_seqlens, ctx.seq_of_token, ctx.slot_ids, act, gates, H, G, D, Dv, taps,
-                     self.spec.unit_eps, float(D) ** -0.5, one_token_each=bool(ctx.decode and ctx.max_q_len == 1))
+                     self.spec.unit_eps, float(D) ** -0.5, one_token_each=one_each)
         o = ctx.buffer("delta_readout", (T, H * Dv), torch.float32)
         y = ctx.buffer("delta_out", (T, H * Dv), self.dtype)
         K.delta_recurrence(act, gates, state, ctx.cu_seqlens, ctx.slot_ids, o, gate, off_gate, self.norm_w, y,
-                           H, G, D, Dv, taps, self.spec.norm_eps, decay=decay, gate_act=self.gate_act)
+                           H, G, D, Dv, taps, self.spec.norm_eps, decay=decay, gate_act=self.gate_act, one_token_each=one_each)
         ops.linear(y, self.w_o, x, epilogue, ctx, col_scale=self.out_scale)
 
 
