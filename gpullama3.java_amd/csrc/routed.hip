@@ -38,8 +38,10 @@ struct RouteExtras {
   float weight_scale;
 };
 
-// Rule 1 by a whole wave: lane l holds the scores of the experts l, l + 64, ...; c: this wave's share of shared memory,
-// E choice scores and n_groups group scores.
+// Rule 1 by a whole wave: lane l works for the experts l, l + 64, ... c: this wave's share of shared memory, E scores, n_groups
+// group scores, and ROUTE_MAX_TOP chosen scores and numbers. Nothing is passed from lane to lane: every lane reads what the
+// others wrote. Up to 256 experts are chosen by rank (a lane counts the experts in front of its own), more by one search for
+// the largest after the other.
 __device__ __forceinline__ void wave_argmax(float& v, int& i) {      // the largest v, of equal ones the lowest i
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) {
@@ -56,66 +58,106 @@ __device__ __forceinline__ void wave_lds_order() {
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
+// how many of the n values stand in front of value v with number i
+__device__ __forceinline__ int rank_among(const float* c, int n, float v, int i) {
+  int r = 0;
+#pragma unroll 4
+  for (int e = 0; e < n; ++e) r += c[e] > v || (c[e] == v && e < i);
+  return r;
+}
+#define ROUTE_BY_RANK 256
+#define ROUTE_WAVE_FLOATS(E, groups) ((E) + (groups) + 2 * ROUTE_MAX_TOP)
 __device__ __forceinline__ void route_choose_scores(const float* __restrict__ logits, int t, int E, int top, int* idx,
                                                     float* __restrict__ wts, int always, const float* __restrict__ correction,
                                                     float sum_eps, const RouteExtras& x, float inv_rms, float* c) {
   const float* z = logits + (long)t * x.ld;
-  const int lane = threadIdx.x & 63, stride = top + (always >= 0 ? 1 : 0);
-  float z_max = -INFINITY, z_sum = 0.f;
-  for (int e = lane; e < E; e += 64) z_max = fmaxf(z_max, z[e]);
-  z_max = wave_max(z_max);
-  for (int e = lane; e < E; e += 64) z_sum += expf(z[e] - z_max);
-  z_sum = wave_sum(z_sum);
+  const int lane = threadIdx.x & 63, stride = top + (always >= 0 ? 1 : 0), per = E / x.n_groups;
+  float* gs = c + E;
+  float* chosen_s = gs + x.n_groups;
+  int* chosen_e = reinterpret_cast<int*>(chosen_s + ROUTE_MAX_TOP);
+  const bool by_rank = E <= ROUTE_BY_RANK;
+  float s[ROUTE_BY_RANK / 64];             // the scores of this lane's experts, where they are few
   wave_lds_order();                        // (the wave's last token is done with its share)
-  for (int e = lane; e < E; e += 64) c[e] = expf(z[e] - z_max) / z_sum + (correction ? correction[e] : 0.f);
+  if (lane < top) {                        // (no number among the scores: any experts, but some that exist)
+    chosen_s[lane] = 0.f;
+    chosen_e[lane] = lane;
+  }
+  float z_max = -INFINITY, z_sum = 0.f;
+  for (int e = lane; e < E; e += 64) c[e] = z[e];
+  wave_lds_order();
+  if (by_rank) {
+#pragma unroll 4
+    for (int e = 0; e < E; ++e) z_max = fmaxf(z_max, c[e]);
+    wave_lds_order();
+#pragma unroll
+    for (int n = 0; n < ROUTE_BY_RANK / 64; ++n)
+      if (lane + 64 * n < E) c[lane + 64 * n] = s[n] = expf(c[lane + 64 * n] - z_max);
+    wave_lds_order();
+#pragma unroll 4
+    for (int e = 0; e < E; ++e) z_sum += c[e];
+    wave_lds_order();
+#pragma unroll
+    for (int n = 0; n < ROUTE_BY_RANK / 64; ++n)
+      if (lane + 64 * n < E) {
+        s[n] /= z_sum;
+        c[lane + 64 * n] = s[n] + (correction ? correction[lane + 64 * n] : 0.f);
+      }
+  } else {
+    for (int e = lane; e < E; e += 64) z_max = fmaxf(z_max, c[e]);
+    z_max = wave_max(z_max);
+    for (int e = lane; e < E; e += 64) z_sum += expf(c[e] - z_max);
+    z_sum = wave_sum(z_sum);
+    for (int e = lane; e < E; e += 64) c[e] = expf(c[e] - z_max) / z_sum + (correction ? correction[e] : 0.f);
+  }
   wave_lds_order();
   if (x.n_groups > 1) {
-    float* gs = c + E;
-    const int per = E / x.n_groups;
     for (int g = lane; g < x.n_groups; g += 64) {
       float m = -INFINITY;
       for (int i = 0; i < per; ++i) m = fmaxf(m, c[g * per + i]);
       gs[g] = m;
     }
-    unsigned open = 0;                     // bit i: group lane + 64 i stays open (at most 16 of them a lane)
-    for (int n = 0; n < x.keep; ++n) {
-      float v = -INFINITY;
-      int best = 0x7fffffff;
-      for (int g = lane, i = 0; g < x.n_groups; g += 64, ++i)
-        if (!(open >> i & 1u) && (best == 0x7fffffff || gs[g] > v)) {
-          v = gs[g];
-          best = g;
-        }
-      wave_argmax(v, best);
-      if (best < x.n_groups && (best & 63) == lane) open |= 1u << (best >> 6);
-    }
-    for (int g = lane, i = 0; g < x.n_groups; g += 64, ++i)
-      if (!(open >> i & 1u))
-        for (int e = 0; e < per; ++e) c[g * per + e] = -INFINITY;
+    wave_lds_order();
+    for (int g = lane; g < x.n_groups; g += 64)
+      if (rank_among(gs, x.n_groups, gs[g], g) >= x.keep)
+        for (int i = 0; i < per; ++i) c[g * per + i] = -INFINITY;
     wave_lds_order();
   }
-  float sum = 0.f, mine = 0.f;             // lane j keeps the score of choice j
-  for (int j = 0; j < top; ++j) {
-    float v = -INFINITY;
-    int best = 0x7fffffff;
-    for (int e = lane; e < E; e += 64)
-      if (c[e] > v) {
-        v = c[e];
-        best = e;
+  if (by_rank) {
+#pragma unroll
+    for (int n = 0; n < ROUTE_BY_RANK / 64; ++n) {
+      const int e = lane + 64 * n;
+      if (e < E && c[e] > -INFINITY) {
+        const int rank = rank_among(c, E, c[e], e);
+        if (rank < top) {
+          chosen_s[rank] = s[n];
+          chosen_e[rank] = e;
+        }
       }
-    wave_argmax(v, best);
-    if (best >= E) best = j;               // (no number among the scores: any expert, but one that exists)
-    const float s = expf(z[best] - z_max) / z_sum;
-    sum += s;
-    if (lane == j) {
-      mine = s;
-      idx[(long)t * stride + j] = best;
     }
-    if ((best & 63) == lane) c[best] = -INFINITY;
+  } else {
+    for (int j = 0; j < top; ++j) {
+      float v = -INFINITY;
+      int best = 0x7fffffff;
+      for (int e = lane; e < E; e += 64)
+        if (c[e] > v) {
+          v = c[e];
+          best = e;
+        }
+      wave_argmax(v, best);
+      if (best < E && (best & 63) == lane) {
+        chosen_s[j] = expf(z[best] - z_max) / z_sum;
+        chosen_e[j] = best;
+        c[best] = -INFINITY;
+      }
+    }
   }
+  wave_lds_order();
+  float sum = 0.f;
+  for (int j = 0; j < top; ++j) sum += chosen_s[j];
   sum += sum_eps;
   if (lane < top) {
-    const float w = mine / sum * x.weight_scale;
+    const float w = chosen_s[lane] / sum * x.weight_scale;
+    idx[(long)t * stride + lane] = chosen_e[lane];
     wts[(long)t * stride + lane] = x.in_wts ? 1.0f : w;
     if (x.in_wts) x.in_wts[(long)t * stride + lane] = w * inv_rms;
   }
@@ -191,10 +233,10 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
 __global__ __launch_bounds__(256) void route_scores_kernel(const float* __restrict__ logits, int T, int E, int top,
                                                            int* __restrict__ idx, float* __restrict__ wts, int always,
                                                            const float* __restrict__ correction, float sum_eps, RouteExtras x) {
-  extern __shared__ float route_lds[];      // per wave E + n_groups
+  extern __shared__ float route_lds[];      // ROUTE_WAVE_FLOATS a wave
   const int wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
   if (t < T)
-    route_choose_scores(logits, t, E, top, idx, wts, always, correction, sum_eps, x, 1.0f, route_lds + wave * (E + x.n_groups));
+    route_choose_scores(logits, t, E, top, idx, wts, always, correction, sum_eps, x, 1.0f, route_lds + wave * ROUTE_WAVE_FLOATS(E, x.n_groups));
 }
 
 // ----------------------------------------------------------------- pairs ordered by expert
@@ -234,7 +276,7 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
                                                           int* __restrict__ offsets, int* __restrict__ sorted, int always,
                                                           int scores, const float* __restrict__ correction, float sum_eps,
                                                           RouteExtras x, int choosers) {
-  extern __shared__ float route_lds[];      // rule 1: E + n_groups floats for each of the `choosers` waves
+  extern __shared__ float route_lds[];      // rule 1: ROUTE_WAVE_FLOATS for each of the `choosers` waves
   __shared__ float inv_rms[64];
   if (x.ssq) {                              // (the same for all threads) a wave a row adds up its partial sums
     for (int t = threadIdx.x >> 6; t < T; t += blockDim.x >> 6) {
@@ -250,7 +292,7 @@ __global__ __launch_bounds__(1024) void route_few_kernel(const float* __restrict
     if (wave < choosers)
       for (int t = wave; t < T; t += choosers)
         route_choose_scores(logits, t, E, top, idx, wts, always, correction, sum_eps, x, x.ssq ? inv_rms[t] : 1.0f,
-                            route_lds + wave * (E + x.n_groups));
+                            route_lds + wave * ROUTE_WAVE_FLOATS(E, x.n_groups));
   } else if ((int)threadIdx.x < T) {
     route_choose(logits, threadIdx.x, E, top, idx, wts, always, scores, x, x.ssq ? inv_rms[threadIdx.x] : 1.0f);
   }
@@ -281,7 +323,7 @@ extern "C" int gl3_route(const float* logits, int n_tokens, int E, int top, int*
                                                   top <= keep * (E / n_groups))),
               "gl3_route: the %d largest of %d experts in the best %d of %d groups", top, E, keep, n_groups);
   const RouteExtras x{ld, in_wts, gate_col, gate_out, ssq, n_partials, d, eps, norm_out, n_groups, keep, weight_scale};
-  const size_t per_wave = (size_t)(E + n_groups) * sizeof(float);
+  const size_t per_wave = (size_t)ROUTE_WAVE_FLOATS(E, n_groups) * sizeof(float);
   if (n_tokens <= 64) {
     int choosers = (int)(40 * 1024 / per_wave);      // (beside the counters of the ordering)
     choosers = choosers > 16 ? 16 : choosers;

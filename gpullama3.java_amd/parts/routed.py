@@ -175,7 +175,7 @@ class RoutedFeedForward:
                 norm = (h.ssq, h.n_partials, d, h.eps)
             else:
                 h = h.materialize()
-        if T > 64 and mfma and h.dtype == self.w_router.dtype == torch.bfloat16 and self.w_router.shape[0] <= 64:
+        if T > ops.FUSE_ROWS and mfma and h.dtype == self.w_router.dtype == torch.bfloat16 and self.w_router.shape[0] <= 64:
             # many rows and few columns: the experts' kernel that slices K (the tiled product would have a block for 128 rows)
             K.expert_gemm(h, self.w_router.unsqueeze(0), logits, mfma=True)
         else:
