@@ -22,7 +22,8 @@ config.json: ``architecture`` "Banazen", ``vocab``, ``width``, ``norm.eps``, ``e
   parallel:      ``left``: ``heads``, ``kv_heads``, ``dim``, ``vdim``, ``conv``, ``rot``: ``base``, ``dims`` (absent: none),
                  ``scale``; ``right``: ``heads``, ``kv_heads``, ``dim``, ``vdim``, ``conv``;
   mlp:           ``{"kind": "dense", "ff"}`` or ``{"kind": "moe", "router": {"experts", "top", "scale", "groups": {"count",
-                 "keep"}}, "expert": {"ff", "limit"}, "shared": {"ff", "limit"} | null}``.
+                 "keep"}}, "expert": {"ff", "limit"}, "shared": {"ff", "limit"} | null}``; without ``scale``, ``groups`` or
+                 ``limit`` (absent or null) there is none.
 The folder names no longest sequence: ``max_positions`` (ours, optional) bounds it, else ``DEFAULT_MAX_POSITIONS``.
 Tensor names: ``embed``, ``side.embed``, ``final.norm``, ``head``, and per layer i ``l<i>.norm1``, ``l<i>.mix.*``,
 ``l<i>.mlp.*``, ``l<i>.side.*``.
@@ -118,7 +119,8 @@ def _check_mlp(mlp, where):
         return
     r, w = mlp.get("router"), where + "router: "
     experts, top = _int(r, "experts", w), _int(r, "top", w)
-    _number(r, "scale", w)
+    if r.get("scale") is not None:
+        _number(r, "scale", w)
     can = experts
     if r.get("groups") is not None:
         count, keep = _int(r["groups"], "count", w + "groups: "), _int(r["groups"], "keep", w + "groups: ")
@@ -129,7 +131,9 @@ def _check_mlp(mlp, where):
         raise ConfigError(f"config.json: {w}the {top} largest of {can} experts")
     for k in ("expert", "shared"):
         if k == "expert" or mlp.get(k) is not None:
-            _int(mlp.get(k), "ff", where + k + ": "), _positive(mlp[k], "limit", where + k + ": ")
+            _int(mlp.get(k), "ff", where + k + ": ")
+            if mlp[k].get("limit") is not None:
+                _positive(mlp[k], "limit", where + k + ": ")
 
 
 @dataclass(frozen=True)
@@ -276,7 +280,8 @@ class BanazenConfiguration:
                                         names={k: q + k for k in ("gate", "up", "down")})
 
         def expert(e):
-            return ExpertSpec(e["ff"], EXPERT_ACTIVATION, gated=True, limit=float(e["limit"]), up_shift=EXPERT_UP_SHIFT)
+            return ExpertSpec(e["ff"], EXPERT_ACTIVATION, gated=True, limit=float(e["limit"]) if e.get("limit") is not None else None,
+                              up_shift=EXPERT_UP_SHIFT)
 
         names = {"router": q + "router", "correction": q + "correction", "expert_gate": q + "e{e}.gate",
                  "expert_up": q + "e{e}.up", "expert_down": q + "e{e}.down"}
@@ -289,7 +294,8 @@ class BanazenConfiguration:
         return RoutedFeedForwardSpec(
             hidden=self.width, n_experts=r["experts"], top=r["top"], expert=expert(mlp["expert"]),
             shared=expert(shared) if shared is not None else None, names=names, weights="scores", sum_eps=ROUTER_SUM_EPS,
-            groups=(groups["count"], groups["keep"]) if groups is not None else None, weight_scale=float(r["scale"]))
+            groups=(groups["count"], groups["keep"]) if groups is not None else None,
+            weight_scale=float(r["scale"]) if r.get("scale") is not None else 1.0)
 
     def model_spec(self):
         def norm(name):
