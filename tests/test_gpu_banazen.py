@@ -338,7 +338,7 @@ def routed(K, logits, top, E, always=False, gate_col=None, **kw):
 
 
 @pytest.mark.parametrize("T", [1, 7, 64, 65, 300])
-@pytest.mark.parametrize("E, top, count, keep", [(6, 2, 3, 2), (8, 4, 4, 3), (9, 4, 3, 2), (8, 3, 8, 5), (64, 6, 8, 2), (256, 8, 8, 4), (130, 5, 65, 3),
+@pytest.mark.parametrize("E, top, count, keep", [(6, 2, 3, 2), (12, 4, 4, 3), (9, 4, 3, 2), (8, 3, 8, 5), (64, 6, 8, 2), (256, 8, 8, 4), (130, 5, 65, 3),
                                                  (1, 1, 1, 1), (5, 5, 1, 1), (1024, 16, 512, 100)])
 def test_router_with_groups(T, E, top, count, keep):
     """Choice scores may be negative (a closed group's experts still count as less than any of them), ties go to the lower
