@@ -141,8 +141,8 @@ class AttentionSpec:
     query_temperature: Optional[QueryTemperature] = None
     value_mix: Optional[ValueMix] = None
     conv_taps: int = 0                # n: each channel of q, k and v passes a causal convolution over time right behind its
-                                      # projection, ``y_t = sum_j w[:, j] u_(t - n + 1 + j)`` with zeros before the sequence's
-                                      # start (names ``q_conv``, ``k_conv``, ``v_conv``: [channels, n]); 0: none
+                                      # projection: channel c of a token becomes ``w[c, n - 1] u[t] + w[c, n - 2] u[t - 1] + ...`` over
+                                      # the sequence's last n projected values u, as far as it has them (names ``q_conv``, ``k_conv``, ``v_conv``: [channels, n]); 0: none
     # (a name ``gate`` among ``names``: a stored [n_heads * v_head_dim, hidden] matrix; the heads' outputs together are
     # multiplied element by element with sigmoid of its product with the mixer's input, before the output projection)
     # (a name ``sink`` among ``names``: a stored [n_heads] vector, a learned sink per query head in place of ``sink``)
@@ -270,9 +270,9 @@ class GatedDeltaSpec:
     """The gated delta rule: per value head a matrix [key_dim, value_dim] in 32-bit that every token decays,
     corrects towards its value along its key, and reads with its query (``parts/delta.py``). ``n_heads`` value
     heads share ``n_kv_heads`` query/key heads; q, k and v pass a causal convolution of ``conv_taps`` taps. With a
-    ``decay_rank`` every row of a head's matrix decays by itself, ``exp(-exp(A_log_h) softplus(W_a2 (W_a1 h) +
-    dt_bias))`` with names ``a1`` [rank, hidden], ``a2`` and ``dt_bias`` over heads x key_dim in place of ``a``; with a
-    ``gate_rank`` the read-out's gate is ``W_g2 (W_g1 h)`` (names ``g1``, ``g2`` in place of ``g``)."""
+    ``decay_rank`` every row of a head's matrix decays by itself: what is added to its ``dt_bias`` is ``a2 @ (a1 @ h)`` (names
+    ``a1`` [rank, hidden], ``a2`` and ``dt_bias`` over heads x key_dim in place of ``a``); with a ``gate_rank`` the read-out's
+    gate is ``g2 @ (g1 @ h)`` (names ``g1``, ``g2`` in place of ``g``)."""
     kind: str = "gated_delta"
     hidden: int = 0
     n_heads: int = 0
@@ -336,7 +336,7 @@ class RoutedFeedForwardSpec:
     # sum plus ``sum_eps``. "chosen_softmax": the softmax over the chosen logits alone.
     weights: str = "chosen_softmax"
     sum_eps: float = 0.0
-    # (with "scores") the experts form ``groups[0]`` equal groups of neighbours, of which the ``groups[1]`` whose largest
+    # (with "scores") experts that follow one another are grouped, ``groups[0]`` equal groups, of which the ``groups[1]`` whose largest
     # choice score is largest stay open; only their experts can be chosen. None: all are open
     groups: Optional[tuple] = None
     weight_scale: float = 1.0         # a constant on the chosen experts' weights (not on the shared expert's)
@@ -354,7 +354,7 @@ class RoutedFeedForwardSpec:
 class TokenSideSpec:
     """What a token's own row of a side table adds behind a layer's sublayers (``parts/token_side.py``): with e the
     columns ``index * dim ..`` of row ``token`` of the stored table ``embed`` [``rows``, ``columns``],
-    ``g = act(W_gate x) * e; y = W_proj g; x <- x + y / rms(y) * norm`` (eps inside the root). x is the residual row itself."""
+    ``x += norm * unit(W_proj (act(W_gate x) * e))``, unit(y) = y over its root mean square (eps inside the root). x is the residual row itself."""
     kind: str = "token_side"
     hidden: int = 0
     dim: int = 0

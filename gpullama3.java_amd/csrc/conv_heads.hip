@@ -3,7 +3,7 @@
 //
 // rows [T][ld]: a token's projected heads, queries (Hq heads of hs elements), keys (Kh of hs), values (Kh of vd), head
 // sizes padded to multiples of 16 with zeros; C = (Hq + Kh) hs + Kh vd channels from column 0 on. Per channel
-//   y_t = sum_j w[j] u_(t - taps + 1 + j),   u before a sequence's start = 0,
+//   y[t] = w[taps - 1] u[t] + w[taps - 2] u[t - 1] + ...,   as far back as the sequence reaches,
 // w [taps][C] float (the last row is the current token's). The inputs before a step's first token are what the sequence's
 // slot holds: `held` [taps - 1][C] floats, oldest first, from `held_off` of the slot's state.
 // Queries and keys: the pairs (2i, 2i + 1) of a head's first `rot` elements are turned by the token's position (tables

@@ -19,7 +19,8 @@
 // weight shared by the heads, times silu or sigmoid of a gate).
 //
 // A decay per key channel instead of one per head: S <- diag(g) S, g of D numbers a head and token. delta_inner makes
-// them, and the read-out's gate, from two-step projections: g = exp(-exp(A_log[h]) softplus(W_a2 (W_a1 h) + dt_bias)).
+// them, and the read-out's gate, from two-step projections: a of a key channel is its row of a second matrix times what a
+// first one made of the input (a few numbers a token), and so is the gate.
 #include "common.h"
 
 __device__ __forceinline__ float dr_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }

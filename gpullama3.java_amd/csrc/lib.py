@@ -834,7 +834,7 @@ def route(logits, top, idx, wts, offsets, pairs, always=False, scores=False, cor
     (``always``), and to ``gate_out`` [T] where given. ``norm = (ssq, n_partials, d, eps)`` (at most 64 tokens, with
     ``in_wts``): the rows that the experts multiply lack their 1 / rms, which is made from the partial sums of squares,
     rides in ``in_wts`` and goes to ``norm_out`` [T] where given. ``groups = (count, keep)`` (with ``scores``): the experts
-    form ``count`` equal groups of neighbours, of which those with the ``keep`` largest choice scores stay open.
+    are grouped as they follow one another, ``count`` equal groups, of which those with the ``keep`` largest choice scores stay open.
     ``weight_scale`` multiplies the chosen experts' weights."""
     _dev(logits, "logits", torch.float32)
     T, ld = logits.shape
@@ -1379,7 +1379,8 @@ def side_gate(x, w, table, col, ids, out, act="gelu_tanh", mfma=True):
 
 
 def norm_add_next(x, y, w, eps, next_weight=None, next_eps=0.0, h=None, xg=None, ssq=None):
-    """``x += y / sqrt(mean(y^2) + eps) * w`` (float32 rows of a multiple of 4 elements), and of the completed rows what the
+    """``x += w * unit(y)``, unit(y) = y over its root mean square with ``eps`` inside the root (float32 rows of a multiple of 4
+    elements), and of the completed rows what the
     norm that reads them next makes: ``h`` = row / sqrt(mean(row^2) + next_eps) * next_weight in h's type, and/or ``xg``
     bfloat16 = next_weight * row with ``ssq`` (at least 64 floats, at most 64 rows) the rows' sums of squares."""
     _dev(x, "x", torch.float32); _dev(y, "y", torch.float32); _dev(w, "w", torch.float32)

@@ -22,8 +22,8 @@
 // [T] where it has no pair. ssq (not null): the rows that the experts will multiply are not normed yet; [n_partials][64]
 // partial sums of squares of the residual rows (at most 64 of them), from which 1 / sqrt(sum / d + eps) is made and
 // multiplied into in_wts (for a pair whose weight is 1 too) and handed out as norm_out [T].
-// n_groups > 1 (rule 1): the experts form that many equal groups of neighbours; a group's score is the largest choice
-// score in it, and only the experts of the `keep` best groups can be chosen (the lower number wins a tie). weight_scale
+// n_groups > 1 (rule 1): of every E / n_groups experts in a row the best one speaks for all; the `keep` groups whose speakers
+// stand first stay open, the others' experts are out of the choice (the lower number wins a tie). weight_scale
 // multiplies the chosen experts' weights.
 struct RouteExtras {
   int ld;

@@ -1,5 +1,5 @@
 // What a token's own row of a side table adds behind a layer's sublayers:
-//   g = act(W_gate x) * e;   y = W_proj g;   x <- x + y / sqrt(mean(y^2) + eps) * w
+//   x += w * unit(W_proj g),   g = act(W_gate x) * e,   unit(y) = y over its root mean square (eps inside the root)
 // x: the 32-bit residual row itself, e: the layer's columns of the token's row. Two kernels; the product with W_proj stands
 // between them.
 //   gl3_side_gate      g in the activations' type, padded with zeros to whole steps of the next product

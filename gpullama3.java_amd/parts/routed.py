@@ -15,7 +15,7 @@ What a description may change: gated experts (``ExpertSpec.gated``: gate and up 
 grouped product's epilogue finds a gate value and its up value in neighbouring lanes and writes
 ``act(min(gate, limit)) * (clamp(up) + shift)`` directly); the other rule for choice and weights (``weights =
 "scores"``: a softmax over all router outputs, the choice by score plus a stored correction, the weights from the
-chosen scores over their sum; ``groups``: only experts of the best groups of neighbours can be chosen; ``weight_scale``: a
+chosen scores over their sum; ``groups``: only experts of the groups whose best choice scores are largest stay open; ``weight_scale``: a
 constant on the chosen experts' weights); the third (``weights = "sigmoid"``: the largest router outputs, each weighted with
 its own sigmoid); a weight that multiplies the expert's input instead of its output (``weight_on``: up and gate rows are
 linear, so the factor goes onto a pair's sums in front of the activation); a shared expert whose output is multiplied

@@ -1,6 +1,6 @@
 """What a token's own row of a side table adds to the residual row behind a layer's sublayers.
 
-    g = act(W_gate x) * e;   y = W_proj g;   x <- x + y / sqrt(mean(y^2) + eps) * w
+    x += w * unit(W_proj g),   g = act(W_gate x) * e,   unit(y) = y over its root mean square (eps inside the root)
 
 x is the residual row itself (whole: sums of the product before it are settled first), e the columns of this layer in the
 token's row of a table that all layers share. Three launches: the first product reads the 32-bit rows and ends with
